@@ -97,6 +97,9 @@ class ScheduleEntry:
     # the embedding output (the rows as they were before the first entry ran) is added to the residual rows
     # right before this entry runs: a stack that passes some layers several times feeds the input in again
     adds_embedding: bool = False
+    # name of the part of `ModelSpec.input_joins` that rewrites the residual rows from themselves and the embedding
+    # output right before this entry runs
+    input_join: Optional[str] = None
 
 
 @dataclass(frozen=True)
@@ -120,6 +123,10 @@ class ModelSpec:
     bos_token_id: Optional[int] = None
     # tensor-name prefix of a position encoding's tensors, by the encoding's name (absent: "position.<name>.")
     position_prefixes: Dict[str, str] = field(default_factory=dict)
+    # joins of the residual rows with the embedding output by name (`ScheduleEntry.input_join`), and the tensor-name prefix
+    # of each one's tensors (absent: "join.<name>.")
+    input_joins: Dict[str, PartSpec] = field(default_factory=dict)
+    input_join_prefixes: Dict[str, str] = field(default_factory=dict)
     # tensors a checkpoint may carry that no part reads (a norm in front of a feed-forward the layer does not have)
     optional_tensors: List[str] = field(default_factory=list)
 

@@ -111,10 +111,11 @@ extern "C" int br_rmsnorm(const float* x, const float* w, void* y, int y_is_bf16
 // reduced by a fixed tree.  `center` 0 leaves the mean out: the RMS norm.  `rows` gathers as in
 // the RMS norm above.  With `add` the normed row is added to the float row `y` instead of
 // stored: y += norm(x) * w, the sum of a branch whose output is normed before it joins the
-// residual rows.
+// residual rows.  `plain` leaves the norm out altogether: y = x * w, or y += x * w with `add` (a branch whose
+// output is scaled channel by channel before it joins the residual rows).
 template <typename T, bool ADD>
 __global__ void layernorm_kernel(const float* __restrict__ x, const float* __restrict__ w, T* __restrict__ y,
-                                 const int* __restrict__ rows, int H, float eps, int center) {
+                                 const int* __restrict__ rows, int H, float eps, int center, int plain) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const float* xr = x + (size_t)(rows ? rows[r] : r) * H;
@@ -125,9 +126,12 @@ __global__ void layernorm_kernel(const float* __restrict__ x, const float* __res
         for (int i = threadIdx.x; i < H; i += blockDim.x) sm += xr[i];
         mean = block_sum(sm, scratch) / (float)H;
     }
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < H; i += blockDim.x) { const float v = xr[i] - mean; ss += v * v; }
-    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
+    float inv = 1.0f;
+    if (!plain) {
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < H; i += blockDim.x) { const float v = xr[i] - mean; ss += v * v; }
+        inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
+    }
     for (int i = threadIdx.x; i < H; i += blockDim.x) {
         const float v = (xr[i] - mean) * inv * w[i];
         if (ADD) yr[i] = from_f32<T>(to_f32<T>(yr[i]) + v);
@@ -141,7 +145,7 @@ __global__ void layernorm_kernel(const float* __restrict__ x, const float* __res
 // behind one half of a layer and the norm in front of the next in one pass over the row.
 template <typename T, typename T2, bool ADD, int VPT>
 __global__ void layernorm_vec_kernel(const float* __restrict__ x, const float* __restrict__ w, T* __restrict__ y,
-                                     const int* __restrict__ rows, int H, float eps, int center,
+                                     const int* __restrict__ rows, int H, float eps, int center, int plain,
                                      const float* __restrict__ w2, T2* __restrict__ y2, float eps2, int center2) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -166,7 +170,7 @@ __global__ void layernorm_vec_kernel(const float* __restrict__ x, const float* _
             for (int e = 0; e < 4; ++e) { v[j][e] -= mean; ss += v[j][e] * v[j][e]; }
         }
     }
-    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
+    const float inv = plain ? 1.0f : 1.0f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
     float sm2 = 0.f;
 #pragma unroll
     for (int j = 0; j < VPT; ++j) {
@@ -229,32 +233,32 @@ __global__ void rows_as_kernel(const float* __restrict__ x, T2* __restrict__ y, 
     if (i < n) y[i] = from_f32<T2>(x[i]);
 }
 extern "C" int br_layernorm(const float* x, const float* w, void* y, int y_is_bf16, const int* rows, int R, int H,
-                            float eps, int center, int add, const float* w2, void* y2, int y2_is_bf16, float eps2,
+                            float eps, int center, int add, int plain, const float* w2, void* y2, int y2_is_bf16, float eps2,
                             int center2, hipStream_t s) {
     if (R <= 0) return BR_OK;
-    if (H <= 0 || (add && (y_is_bf16 || rows)) || (w2 && !y2) || (y2 && !add)) return BR_BAD_ARG;
+    if (H <= 0 || (plain && center) || (add && (y_is_bf16 || rows)) || (w2 && !y2) || (y2 && !add)) return BR_BAD_ARG;
     const int threads = H >= 2048 ? 256 : (H >= 512 ? 128 : 64);
     const bool vec = (H % 4 == 0) && (H / 4 <= 4 * threads) &&
                      (((uintptr_t)x | (uintptr_t)w | (uintptr_t)y | (uintptr_t)w2 | (uintptr_t)y2) % 16 == 0);
     if (vec) {
         if (add) {
-            if (y2_is_bf16) layernorm_vec_kernel<float, bf16, true, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, w2, (bf16*)y2, eps2, center2);
-            else layernorm_vec_kernel<float, float, true, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, w2, (float*)y2, eps2, center2);
-        } else if (y_is_bf16) layernorm_vec_kernel<bf16, float, false, 4><<<R, threads, 0, s>>>(x, w, (bf16*)y, rows, H, eps, center, nullptr, nullptr, 0.f, 0);
-        else layernorm_vec_kernel<float, float, false, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, nullptr, nullptr, 0.f, 0);
+            if (y2_is_bf16) layernorm_vec_kernel<float, bf16, true, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, plain, w2, (bf16*)y2, eps2, center2);
+            else layernorm_vec_kernel<float, float, true, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, plain, w2, (float*)y2, eps2, center2);
+        } else if (y_is_bf16) layernorm_vec_kernel<bf16, float, false, 4><<<R, threads, 0, s>>>(x, w, (bf16*)y, rows, H, eps, center, plain, nullptr, nullptr, 0.f, 0);
+        else layernorm_vec_kernel<float, float, false, 4><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, plain, nullptr, nullptr, 0.f, 0);
         return br_check_launch();
     }
-    if (add) layernorm_kernel<float, true><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center);
-    else if (y_is_bf16) layernorm_kernel<bf16, false><<<R, threads, 0, s>>>(x, w, (bf16*)y, rows, H, eps, center);
-    else layernorm_kernel<float, false><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center);
+    if (add) layernorm_kernel<float, true><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, plain);
+    else if (y_is_bf16) layernorm_kernel<bf16, false><<<R, threads, 0, s>>>(x, w, (bf16*)y, rows, H, eps, center, plain);
+    else layernorm_kernel<float, false><<<R, threads, 0, s>>>(x, w, (float*)y, rows, H, eps, center, plain);
     if (y2 && !w2) {
         const size_t n = (size_t)R * H;
         if (y2_is_bf16) rows_as_kernel<bf16><<<(unsigned)((n + 255) / 256), 256, 0, s>>>((const float*)y, (bf16*)y2, n);
         else rows_as_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, s>>>((const float*)y, (float*)y2, n);
     }
     if (w2) {       // widths the one-pass kernel does not take: the second norm as a launch of its own
-        if (y2_is_bf16) layernorm_kernel<bf16, false><<<R, threads, 0, s>>>((const float*)y, w2, (bf16*)y2, nullptr, H, eps2, center2);
-        else layernorm_kernel<float, false><<<R, threads, 0, s>>>((const float*)y, w2, (float*)y2, nullptr, H, eps2, center2);
+        if (y2_is_bf16) layernorm_kernel<bf16, false><<<R, threads, 0, s>>>((const float*)y, w2, (bf16*)y2, nullptr, H, eps2, center2, 0);
+        else layernorm_kernel<float, false><<<R, threads, 0, s>>>((const float*)y, w2, (float*)y2, nullptr, H, eps2, center2, 0);
     }
     return br_check_launch();
 }
@@ -511,27 +515,64 @@ extern "C" int br_silu_mul(const void* gu, void* a, int is_bf16, int T, int I, h
 
 // ----------------------------------------------------------- clamped gated unit -----
 // a[t, i] = g sigmoid(alpha g) (u + 1) with g = min(gu[t, i] + b[i], limit) and
-// u = clamp(gu[t, I + i] + b[I + i], -limit, limit), from the float sums gu [T, 2 I] of the fused gate/up
-// product and their biases b [2 I] (null: none); a has the products' type.
-template <typename T>
-__global__ void clamped_glu_kernel(const float* __restrict__ gu, const float* __restrict__ b, T* __restrict__ a,
-                                   int I, size_t n, float limit, float alpha) {
-    size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+// u = clamp(gu[t, I + i] + b[I + i], -limit, limit), from the fused gate/up product gu [T, 2 I] (its float sums, or
+// their roundings) and the biases b [2 I] (null: none); a has the products' type.  `row_gate` (null: none): a number a
+// row, `gate_stride` elements apart; the row is multiplied by its sigmoid.  VEC 4: four elements a thread (I in steps
+// of 4, aligned buffers).
+template <typename T> struct ew_vec4;
+template <> struct ew_vec4<float> { typedef f32x4 type; };
+template <> struct ew_vec4<bf16> { typedef bf16x4 type; };
+template <typename T, int VEC>
+__device__ __forceinline__ void ew_load(const T* p, float* v) {
+    if (VEC == 4) {
+        const typename ew_vec4<T>::type q = *(const typename ew_vec4<T>::type*)p;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = to_f32<T>(q[e]);
+    } else v[0] = to_f32<T>(p[0]);
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void ew_store(T* p, const float* v) {
+    if (VEC == 4) {
+        typename ew_vec4<T>::type q;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) q[e] = from_f32<T>(v[e]);
+        *(typename ew_vec4<T>::type*)p = q;
+    } else p[0] = from_f32<T>(v[0]);
+}
+template <typename TG, typename T, int VEC>
+__global__ void clamped_glu_kernel(const TG* __restrict__ gu, const float* __restrict__ b, const float* __restrict__ row_gate,
+                                   size_t gate_stride, T* __restrict__ a, int I, size_t n, float limit, float alpha) {
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= n) return;
-    size_t t = i / I, c = i - t * I;
-    float g = gu[t * 2 * I + c] + (b ? b[c] : 0.f), u = gu[t * 2 * I + I + c] + (b ? b[I + c] : 0.f);
-    g = fminf(g, limit);
-    u = fminf(fmaxf(u, -limit), limit);
-    a[i] = from_f32<T>(g / (1.f + expf(-alpha * g)) * (u + 1.f));
+    const size_t t = i / I, c = i - t * I;
+    const float mul = row_gate ? 1.f / (1.f + expf(-row_gate[t * gate_stride])) : 1.f;
+    float gv[VEC], uv[VEC];
+    ew_load<TG, VEC>(gu + t * 2 * I + c, gv);
+    ew_load<TG, VEC>(gu + t * 2 * I + I + c, uv);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+        const float g = fminf(gv[e] + (b ? b[c + e] : 0.f), limit);
+        const float u = fminf(fmaxf(uv[e] + (b ? b[I + c + e] : 0.f), -limit), limit);
+        gv[e] = g / (1.f + expf(-alpha * g)) * (u + 1.f) * mul;
+    }
+    ew_store<T, VEC>(a + i, gv);
 }
 
-extern "C" int br_clamped_glu(const float* gu, const float* b, void* a, int a_is_bf16, int T, int I, float limit,
-                              float alpha, hipStream_t s) {
+extern "C" int br_clamped_glu(const void* gu, int gu_is_bf16, const float* b, const float* row_gate, size_t gate_stride, void* a,
+                              int a_is_bf16, int T, int I, float limit, float alpha, hipStream_t s) {
     if (T <= 0 || I <= 0) return BR_OK;
-    size_t n = (size_t)T * I;
-    unsigned blocks = (unsigned)((n + 255) / 256);
-    if (a_is_bf16) clamped_glu_kernel<bf16><<<blocks, 256, 0, s>>>(gu, b, (bf16*)a, I, n, limit, alpha);
-    else clamped_glu_kernel<float><<<blocks, 256, 0, s>>>(gu, b, (float*)a, I, n, limit, alpha);
+    if (gu_is_bf16 && !a_is_bf16) return BR_BAD_ARG;
+    const size_t n = (size_t)T * I;
+    const bool vec = I % 4 == 0 && (((uintptr_t)gu | (uintptr_t)a) & 15) == 0;
+    const unsigned blocks = (unsigned)(((vec ? n / 4 : n) + 255) / 256);
+#define CG_GO(TG, TT) do { \
+        if (vec) clamped_glu_kernel<TG, TT, 4><<<blocks, 256, 0, s>>>((const TG*)gu, b, row_gate, gate_stride, (TT*)a, I, n, limit, alpha); \
+        else clamped_glu_kernel<TG, TT, 1><<<blocks, 256, 0, s>>>((const TG*)gu, b, row_gate, gate_stride, (TT*)a, I, n, limit, alpha); \
+    } while (0)
+    if (gu_is_bf16) CG_GO(bf16, bf16);
+    else if (a_is_bf16) CG_GO(float, bf16);
+    else CG_GO(float, float);
+#undef CG_GO
     return br_check_launch();
 }
 
@@ -617,6 +658,34 @@ extern "C" int br_convert(const void* a, void* b, int to_bf16, size_t n, hipStre
     unsigned blocks = (unsigned)((n + 255) / 256);
     if (to_bf16) f32_to_bf16_kernel<<<blocks, 256, 0, s>>>((const float*)a, (bf16*)b, n);
     else bf16_to_f32_kernel<<<blocks, 256, 0, s>>>((const bf16*)a, (float*)b, n);
+    return br_check_launch();
+}
+
+// out[t, i] = x[t, i] for float rows x [T, H], in out's type; out's rows lie `ldo` elements apart (a column range of
+// wider rows).  VEC: four elements a thread (H and ldo in steps of 4, aligned).
+template <typename T, int VEC>
+__global__ void rows_into_kernel(const float* __restrict__ x, T* __restrict__ out, int H, size_t ldo, size_t n) {
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+    if (i >= n) return;
+    const size_t t = i / H, c = i - t * H;
+    float v[VEC];
+    ew_load<float, VEC>(x + i, v);
+    ew_store<T, VEC>(out + t * ldo + c, v);
+}
+
+extern "C" int br_rows_into(const float* x, void* out, int is_bf16, int T, int H, size_t ldo, hipStream_t s) {
+    if (T <= 0) return BR_OK;
+    if (H <= 0 || ldo < (size_t)H) return BR_BAD_ARG;
+    const size_t n = (size_t)T * H;
+    const bool vec = H % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0;
+    const unsigned blocks = (unsigned)(((vec ? n / 4 : n) + 255) / 256);
+    if (is_bf16) {
+        if (vec) rows_into_kernel<bf16, 4><<<blocks, 256, 0, s>>>(x, (bf16*)out, H, ldo, n);
+        else rows_into_kernel<bf16, 1><<<blocks, 256, 0, s>>>(x, (bf16*)out, H, ldo, n);
+    } else {
+        if (vec) rows_into_kernel<float, 4><<<blocks, 256, 0, s>>>(x, (float*)out, H, ldo, n);
+        else rows_into_kernel<float, 1><<<blocks, 256, 0, s>>>(x, (float*)out, H, ldo, n);
+    }
     return br_check_launch();
 }
 

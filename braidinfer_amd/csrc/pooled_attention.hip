@@ -9,7 +9,7 @@
 // key of score 0 without a value, i.e. one added to the denominator.
 //
 // Three kernels: `prepare` (bias, per-head RMS norm of queries and keys, rotation of the
-// first `rd` elements in (i, i + rd/2) pairs, value mixing with another layer's values,
+// first `rd` elements in (i, i + rd/2) or (2i, 2i + 1) pairs, value mixing with another layer's values,
 // cache write), `pool` (the means of the blocks that the step completed) and `attend`.
 // Keys and values of a page: keys [kv_head][token][dk] and, behind the keys of all heads, values
 // transposed, [kv_head][dv][token]: the operand layout of the matrix-core kernel below (a lane reads
@@ -52,6 +52,9 @@ __device__ __forceinline__ int pwa_lo(int p, int size, int chunk) {
 // nq * maps query heads over nkv kv heads whose scores are the maps' own.  `row_ss` [T, 2]: the sums of squares of
 // the token's whole query and key projections (bias included); the norm then runs over the whole projection
 // instead of a head, and `nw_stride` = dk gives every head norm weights of its own (0: one [dk] for all).
+// `adjacent`: elements 2i and 2i + 1 are the pair that turns together (else i and i + rd/2).  `q_scale` (null: none): a
+// factor per query head on its queries, i.e. on all the head's scores.  `v_eps` >= 0: every head's values are divided
+// by their root mean square (no weight) before they are stored.
 template <typename T>
 __global__ __launch_bounds__(64) void pwa_prepare_kernel(
     const float* __restrict__ qkv, const float* __restrict__ bias, const float* __restrict__ qn_w,
@@ -61,7 +64,7 @@ __global__ __launch_bounds__(64) void pwa_prepare_kernel(
     T* __restrict__ q_out, T* __restrict__ storage, float* __restrict__ v_first,
     const float* __restrict__ lambda, int vf_role, int nq, int nkv, int dk, int dv, int page,
     int write_cache, int width, int v_col0, float q_coef, int q_every, int maps, const float* __restrict__ row_ss,
-    int nw_stride, int pad_q) {
+    int nw_stride, int pad_q, int adjacent, const float* __restrict__ q_scale, float v_eps) {
     extern __shared__ float row[];          // [max(dk, dv)]
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int nqs = nq * maps, nks = nkv * maps, kw = maps * dk;     // vectors of dk, and a key row's width
@@ -119,6 +122,15 @@ __global__ __launch_bounds__(64) void pwa_prepare_kernel(
 #pragma unroll
             for (int j = 0; j < MAX_EPL; ++j) v[j] *= temp;
         }
+        if (is_q && q_scale) {
+            const float mul = q_scale[h / maps];
+#pragma unroll
+            for (int j = 0; j < MAX_EPL; ++j) v[j] *= mul;
+        }
+    } else if (v_eps >= 0.f) {
+        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dv + v_eps);
+#pragma unroll
+        for (int j = 0; j < MAX_EPL; ++j) v[j] *= inv;
     }
     if (rd > 0) {                           // the barrier is met whatever the head
         const int half = rd >> 1;
@@ -135,9 +147,11 @@ __global__ __launch_bounds__(64) void pwa_prepare_kernel(
             for (int j = 0; j < MAX_EPL; ++j) {
                 const int i = lane + 64 * j;
                 if (i < rd) {
-                    const int f = i < half ? i : i - half;
+                    const bool second = adjacent ? (i & 1) : i >= half;
+                    const int f = adjacent ? i >> 1 : (second ? i - half : i);
+                    const float other = row[adjacent ? i ^ 1 : (second ? i - half : i + half)];
                     const float c = cs[(size_t)t * half + f], s = sn[(size_t)t * half + f];
-                    v[j] = i < half ? row[i] * c - row[i + half] * s : row[i] * c + row[i - half] * s;
+                    v[j] = second ? row[i] * c + other * s : row[i] * c - other * s;
                 }
             }
         }
@@ -165,14 +179,14 @@ __global__ __launch_bounds__(64) void pwa_prepare_kernel(
 
 // The values of a step of many tokens: a workgroup takes 64 packed tokens x 64 channels of one kv head through
 // an LDS tile, so that the float sums are read in rows (bias, mixing and `v_first` as in `prepare`) and the
-// transposed values are stored 64 neighbouring tokens of a channel at a time.  grid (ceil(T / 64), nkv,
-// ceil(dv / 64)), block 256.
+// transposed values are stored 64 neighbouring tokens of a channel at a time.  `v_eps` as in `prepare`: a wave first
+// sums the squares of its tokens' whole value rows, in `prepare`'s order.  grid (ceil(T / 64), nkv, ceil(dv / 64)), block 256.
 template <typename T>
 __global__ __launch_bounds__(256) void pwa_values_kernel(
     const float* __restrict__ qkv, const float* __restrict__ bias, const int* __restrict__ pos,
     const int* __restrict__ seq_of_token, const int* __restrict__ slots, const int* __restrict__ block_table,
     int table_stride, T* __restrict__ storage, float* __restrict__ v_first, const float* __restrict__ lambda,
-    int vf_role, int n_tokens, int nq, int nkv, int dk, int dv, int page, int width, int v_col0) {
+    int vf_role, int n_tokens, int nq, int nkv, int dk, int dv, int page, int width, int v_col0, float v_eps) {
     // `dk` is the width of a key row of the cache (all maps of a head)
     __shared__ float tile[64][65];
     const int t0 = blockIdx.x * 64, kvh = blockIdx.y, c0 = blockIdx.z * 64;
@@ -190,6 +204,15 @@ __global__ __launch_bounds__(256) void pwa_values_kernel(
                 if (vf_role == 1) *vf = v;
                 else v = (1.0f - lam) * v + lam * *vf;
             }
+        }
+        if (v_eps >= 0.f) {                 // no value mixing with this norm
+            float ss = 0.f;
+            if (t < n_tokens)
+                for (int i = lane; i < dv; i += 64) {
+                    const float u = qkv[(size_t)t * width + col0 + i] + (bias ? bias[col0 + i] : 0.f);
+                    ss += u * u;
+                }
+            v *= 1.0f / sqrtf(wave_sum(ss) / (float)dv + v_eps);
         }
         tile[tt][lane] = v;
     }
@@ -243,9 +266,10 @@ extern "C" int br_pwa_prepare(const float* qkv, const float* bias, const float* 
                               const int* slots, const int* block_table, int table_stride, void* q_out,
                               void* storage, int is_bf16, float* v_first, const float* lambda, int vf_role,
                               int T, int nq, int nkv, int dk, int dv, int page, int write_cache, int width, int v_from_k,
-                              float q_coef, int q_every, int maps, float* row_ss, int nw_stride, int pad_q, hipStream_t s) {
+                              float q_coef, int q_every, int maps, float* row_ss, int nw_stride, int pad_q, int adjacent,
+                              const float* q_scale, float v_eps, hipStream_t s) {
     if (T <= 0) return BR_OK;
-    if (maps <= 0 || (maps > 1 && v_from_k) || (nw_stride != 0 && nw_stride != dk)) return BR_BAD_ARG;
+    if (maps <= 0 || (maps > 1 && v_from_k) || (v_eps >= 0.f && vf_role) || (nw_stride != 0 && nw_stride != dk)) return BR_BAD_ARG;
     const int nqs = nq * maps, nks = nkv * maps, kw = maps * dk;
     const int v_col0 = v_from_k ? nqs * dk : (nqs + nks) * dk;
     if (width < v_col0 + nkv * dv || (v_from_k && dv != dk) || (bias && v_from_k) || q_every < 0) return BR_BAD_ARG;
@@ -266,21 +290,21 @@ extern "C" int br_pwa_prepare(const float* qkv, const float* bias, const float* 
         pwa_prepare_kernel<bf16><<<grid, 64, lds, s>>>(qkv, bias, qn_w, kn_w, eps, cs, sn, rd, pos, seq_of_token, slots,
                                                        block_table, table_stride, (bf16*)q_out, (bf16*)storage, v_first,
                                                        lambda, vf_role, nq, nkv, dk, dv, page, write_cache, width, v_col0, q_coef, q_every,
-                                                       maps, row_ss, nw_stride, pad_q);
+                                                       maps, row_ss, nw_stride, pad_q, adjacent, q_scale, v_eps);
     else
         pwa_prepare_kernel<float><<<grid, 64, lds, s>>>(qkv, bias, qn_w, kn_w, eps, cs, sn, rd, pos, seq_of_token, slots,
                                                         block_table, table_stride, (float*)q_out, (float*)storage,
                                                         v_first, lambda, vf_role, nq, nkv, dk, dv, page, write_cache, width, v_col0, q_coef, q_every,
-                                                        maps, row_ss, nw_stride, pad_q);
+                                                        maps, row_ss, nw_stride, pad_q, adjacent, q_scale, v_eps);
     int rc = br_check_launch();
     if (rc != BR_OK || !tiled) return rc;
     dim3 vgrid((T + 63) / 64, nkv, (dv + 63) / 64);
     if (is_bf16)
         pwa_values_kernel<bf16><<<vgrid, 256, 0, s>>>(qkv, bias, pos, seq_of_token, slots, block_table, table_stride, (bf16*)storage,
-                                                      v_first, lambda, vf_role, T, nq, nkv, kw, dv, page, width, v_col0);
+                                                      v_first, lambda, vf_role, T, nq, nkv, kw, dv, page, width, v_col0, v_eps);
     else
         pwa_values_kernel<float><<<vgrid, 256, 0, s>>>(qkv, bias, pos, seq_of_token, slots, block_table, table_stride, (float*)storage,
-                                                       v_first, lambda, vf_role, T, nq, nkv, kw, dv, page, width, v_col0);
+                                                       v_first, lambda, vf_role, T, nq, nkv, kw, dv, page, width, v_col0, v_eps);
     return br_check_launch();
 }
 

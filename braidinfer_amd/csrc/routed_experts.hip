@@ -11,9 +11,23 @@
 // experts' weights are what a step reads.  Steps of many tokens go expert by expert through the library's matrix
 // products instead: `sort` groups the (token, slot) pairs by expert, `gather` copies their rows into that order,
 // and `combine` adds every token's weighted outputs back in slot order.
+//
+// Identity experts: a chosen number e >= E (E the experts with matrices) stands for an expert whose output is its input
+// row.  Such pairs are sorted into one bin behind the experts', no product sees them, and `down` / `combine` take the
+// row of h itself.  The gated unit may be the clamped one (`alpha` > 0): g sigmoid(alpha g) (u + 1) with
+// g = min(W_g h, limit), u = clamp(W_u h, -limit, limit).
 #include "common.h"
 
 #define RX_MAX_PER_LANE 8          // experts a lane keeps: up to 512 experts
+
+__device__ __forceinline__ float rx_glu(float g, float u, float limit, float alpha) {
+    if (alpha > 0.f) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit);
+        return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+    }
+    return g / (1.0f + expf(-g)) * u;
+}
 
 // grid (T), one wave a token.
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ scores, const float* __restrict__ bias,
@@ -61,19 +75,50 @@ extern "C" int br_route_topk(const float* scores, const float* bias, int* chosen
     return br_check_launch();
 }
 
-// Routing by sigmoid scores with a choice correction and groups of experts.  s = sigmoid(z); the choice is made on
-// c = s + correction, the shares on s.  With `groups` > 1 the experts form that many runs of E / groups neighbours; a
+// A lane's scores s of its router logits z (its outputs lane, lane + 64, ...): sigmoid(z), or with SOFTMAX the softmax
+// over all E outputs.
+template <int NPL, bool SOFTMAX>
+__device__ __forceinline__ void route_scores(const float* __restrict__ zrow, int E, int lane, float* sg) {
+    if (!SOFTMAX) {
+#pragma unroll
+        for (int i = 0; i < NPL; ++i) {
+            const int e = lane + 64 * i;
+            sg[i] = e < E ? 1.0f / (1.0f + expf(-zrow[e])) : 0.f;
+        }
+        return;
+    }
+    float m = -INFINITY, total = 0.f;
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+        const int e = lane + 64 * i;
+        sg[i] = e < E ? zrow[e] : -INFINITY;
+        m = fmaxf(m, sg[i]);
+    }
+    m = wave_max(m);
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) {
+        sg[i] = lane + 64 * i < E ? expf(sg[i] - m) : 0.f;
+        total += sg[i];
+    }
+    total = wave_sum(total);
+#pragma unroll
+    for (int i = 0; i < NPL; ++i) sg[i] /= total;
+}
+
+// Routing by scores with a choice correction and groups of experts.  s = sigmoid(z), or (SOFTMAX) the softmax of z over
+// all outputs; the choice is made on c = s + correction, the shares on s.  A token's logits lie `ld` elements apart.  With `groups` > 1 the experts form that many runs of E / groups neighbours; a
 // run's score is the sum of its two largest c (of its one, where a run is one expert), only experts of the `keep`
 // best runs can be chosen (the others count as minus infinity), ties to the lower number everywhere.  The shares are
-// the chosen experts' s over their sum (+ 1e-20), times `out_scale`.  grid (T), one wave a token.
+// the chosen experts' s over their sum (+ 1e-20), or as they are without `renorm`, times `out_scale`.  grid (T), one wave
+// a token.
 // Nothing is found by rounds of wave-wide maxima: every expert counts the experts that go before it (a larger c, or
 // the same c and a lower number) by reading all c from LDS, and is chosen when fewer than `top` do, its count being
 // its place among the chosen; the runs are kept the same way.  LDS: E + groups + 128 words.
 // NPL: experts (and runs) a lane holds; the launcher takes this kernel up to 64 experts (NPL 1).
-template <int NPL>
-__global__ __launch_bounds__(64) void route_sigmoid_kernel(const float* __restrict__ scores, const float* __restrict__ correction,
-                                                           int* __restrict__ chosen, float* __restrict__ share, int E, int top,
-                                                           int groups, int keep, float out_scale) {
+template <int NPL, bool SOFTMAX>
+__global__ __launch_bounds__(64) void route_corrected_kernel(const float* __restrict__ scores, int ld, const float* __restrict__ correction,
+                                                             int* __restrict__ chosen, float* __restrict__ share, int E, int top,
+                                                             int groups, int keep, int renorm, float out_scale) {
     extern __shared__ float rs_lds[];
     float* cs = rs_lds;                     // [E] the choice scores
     float* gsL = cs + E;                    // [groups] the runs' scores, then whether a run is kept
@@ -81,13 +126,12 @@ __global__ __launch_bounds__(64) void route_sigmoid_kernel(const float* __restri
     int* who = (int*)(picked + 64);         // [64] the chosen experts by their place
     const int t = blockIdx.x, lane = threadIdx.x;
     float sg[NPL], z[NPL];
+    route_scores<NPL, SOFTMAX>(scores + (size_t)t * ld, E, lane, sg);
 #pragma unroll
     for (int i = 0; i < NPL; ++i) {
         const int e = lane + 64 * i;
-        sg[i] = 0.f;
         z[i] = -INFINITY;
         if (e < E) {
-            sg[i] = 1.0f / (1.0f + expf(-scores[(size_t)t * E + e]));
             z[i] = sg[i] + (correction ? correction[e] : 0.f);
             cs[e] = z[i];
         }
@@ -157,7 +201,7 @@ __global__ __launch_bounds__(64) void route_sigmoid_kernel(const float* __restri
     if (lane < top) {
         float total = 0.f;
         for (int s = 0; s < top; ++s) total += picked[s];          // in the order of the places
-        share[(size_t)t * top + lane] = picked[lane] / (total + 1e-20f) * out_scale;
+        share[(size_t)t * top + lane] = (renorm ? picked[lane] / (total + 1e-20f) : picked[lane]) * out_scale;
         chosen[(size_t)t * top + lane] = who[lane];
     }
 }
@@ -165,19 +209,19 @@ __global__ __launch_bounds__(64) void route_sigmoid_kernel(const float* __restri
 // The same for more than 64 experts, where a lane holds several: the kept runs and then the `top` experts are taken one
 // after the other by rounds of wave-wide maxima (counting places would walk every choice score once per expert a lane
 // holds: 51 us at 256 experts against 9).  LDS: E floats.
-__global__ __launch_bounds__(64) void route_sigmoid_rounds_kernel(const float* __restrict__ scores, const float* __restrict__ correction,
-                                                           int* __restrict__ chosen, float* __restrict__ share, int E, int top,
-                                                           int groups, int keep, float out_scale) {
+template <bool SOFTMAX>
+__global__ __launch_bounds__(64) void route_corrected_rounds_kernel(const float* __restrict__ scores, int ld, const float* __restrict__ correction,
+                                                                    int* __restrict__ chosen, float* __restrict__ share, int E, int top,
+                                                                    int groups, int keep, int renorm, float out_scale) {
     extern __shared__ float cs[];           // the choice scores
     const int t = blockIdx.x, lane = threadIdx.x;
     float sg[RX_MAX_PER_LANE], z[RX_MAX_PER_LANE];
+    route_scores<RX_MAX_PER_LANE, SOFTMAX>(scores + (size_t)t * ld, E, lane, sg);
 #pragma unroll
     for (int i = 0; i < RX_MAX_PER_LANE; ++i) {
         const int e = lane + 64 * i;
-        sg[i] = 0.f;
         z[i] = -INFINITY;
         if (e < E) {
-            sg[i] = 1.0f / (1.0f + expf(-scores[(size_t)t * E + e]));
             z[i] = sg[i] + (correction ? correction[e] : 0.f);
             cs[e] = z[i];
         }
@@ -253,18 +297,23 @@ __global__ __launch_bounds__(64) void route_sigmoid_rounds_kernel(const float* _
         for (int i = 0; i < RX_MAX_PER_LANE; ++i)
             if (lane + 64 * i == at) z[i] = -INFINITY;
     }
-    if (lane < top) share[(size_t)t * top + lane] = mine / (total + 1e-20f) * out_scale;
+    if (lane < top) share[(size_t)t * top + lane] = (renorm ? mine / (total + 1e-20f) : mine) * out_scale;
 }
 
-extern "C" int br_route_sigmoid(const float* scores, const float* correction, int* chosen, float* share, int T, int E, int top,
-                                int groups, int keep, float out_scale, hipStream_t s) {
+// `softmax`: s is the softmax over all E outputs, else the sigmoid; `renorm`: the shares are divided by their sum.
+extern "C" int br_route_corrected(const float* scores, int ld, const float* correction, int* chosen, float* share, int T, int E, int top,
+                                  int groups, int keep, int softmax, int renorm, float out_scale, hipStream_t s) {
     if (T <= 0) return BR_OK;
-    if (E <= 0 || E > 64 * RX_MAX_PER_LANE || top <= 0 || top > E || top > 64 || groups <= 0 || E % groups ||
+    if (E <= 0 || E > 64 * RX_MAX_PER_LANE || top <= 0 || top > E || top > 64 || groups <= 0 || E % groups || ld < E ||
         (groups > 1 && (keep <= 0 || keep > groups)))
         return BR_BAD_ARG;
-    const size_t lds = (size_t)(E + groups + 128) * sizeof(float);
-    if (E <= 64) route_sigmoid_kernel<1><<<T, 64, lds, s>>>(scores, correction, chosen, share, E, top, groups, keep, out_scale);
-    else route_sigmoid_rounds_kernel<<<T, 64, (size_t)E * sizeof(float), s>>>(scores, correction, chosen, share, E, top, groups, keep, out_scale);
+    const size_t lds = (size_t)(E + groups + 128) * sizeof(float), lds_rounds = (size_t)E * sizeof(float);
+#define RX_ROUTE(SM) do { \
+        if (E <= 64) route_corrected_kernel<1, SM><<<T, 64, lds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, renorm, out_scale); \
+        else route_corrected_rounds_kernel<SM><<<T, 64, lds_rounds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, renorm, out_scale); \
+    } while (0)
+    if (softmax) RX_ROUTE(true); else RX_ROUTE(false);
+#undef RX_ROUTE
     return br_check_launch();
 }
 
@@ -293,13 +342,15 @@ __device__ __forceinline__ float rx_dot(const T* __restrict__ wrow, const float*
 // grid (T * top, ceil(F / 16)), 4 waves, a wave four columns.  LDS: W floats.
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void experts_up_kernel(const T* __restrict__ h, const T* __restrict__ w_gu,
-                                                         const int* __restrict__ chosen, T* __restrict__ y, int W, int F, int top) {
+                                                         const int* __restrict__ chosen, T* __restrict__ y, int W, int F, int top,
+                                                         int E, float limit, float alpha) {
     extern __shared__ float hs[];
     const int slot = blockIdx.x, t = slot / top;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int e = chosen[slot];
+    if (e >= E) return;                     // an identity expert has no product
     for (int i = threadIdx.x; i < W; i += 256) hs[i] = to_f32<T>(h[(size_t)t * W + i]);
     __syncthreads();
-    const int e = chosen[slot];
     const T* wg = w_gu + (size_t)e * 2 * F * W;
     const T* wu = wg + (size_t)F * W;
     for (int j = 0; j < 4; ++j) {
@@ -307,7 +358,7 @@ __global__ __launch_bounds__(256) void experts_up_kernel(const T* __restrict__ h
         if (f >= F) break;
         const float g = rx_dot<T, VEC>(wg + (size_t)f * W, hs, W, lane);
         const float u = rx_dot<T, VEC>(wu + (size_t)f * W, hs, W, lane);
-        if (lane == 0) y[(size_t)slot * F + f] = from_f32<T>(g / (1.0f + expf(-g)) * u);
+        if (lane == 0) y[(size_t)slot * F + f] = from_f32<T>(rx_glu(g, u, limit, alpha));
     }
 }
 
@@ -315,7 +366,8 @@ __global__ __launch_bounds__(256) void experts_up_kernel(const T* __restrict__ h
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__ y, const T* __restrict__ w_down,
                                                            const int* __restrict__ chosen, const float* __restrict__ share,
-                                                           float* __restrict__ x, int W, int F, int top) {
+                                                           const T* __restrict__ h, float* __restrict__ x, int W, int F, int top,
+                                                           int E, int store) {
     extern __shared__ float ys[];
     const int t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -327,35 +379,39 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
         float sum = 0.f;
         for (int s = 0; s < top; ++s) {
             const int e = chosen[(size_t)t * top + s];
-            const float d = rx_dot<T, VEC>(w_down + ((size_t)e * W + n) * F, ys + (size_t)s * F, F, lane);
+            const float d = e < E ? rx_dot<T, VEC>(w_down + ((size_t)e * W + n) * F, ys + (size_t)s * F, F, lane)
+                                  : to_f32<T>(h[(size_t)t * W + n]);
             sum = fmaf(share[(size_t)t * top + s], d, sum);
         }
-        if (lane == 0) x[(size_t)t * W + n] += sum;
+        if (lane == 0) x[(size_t)t * W + n] = store ? sum : x[(size_t)t * W + n] + sum;
     }
 }
 
+// Chosen numbers from E on are identity experts (their y is not written); `alpha` > 0: the clamped unit.
 extern "C" int br_experts_up(const void* h, const void* w_gu, const int* chosen, void* y, int is_bf16,
-                             int T, int W, int F, int top, hipStream_t s) {
+                             int T, int W, int F, int top, int E, float limit, float alpha, hipStream_t s) {
     if (T <= 0) return BR_OK;
     if (W <= 0 || F <= 0 || top <= 0 || (size_t)W * 4 > 65536 || (F + 15) / 16 > 65535) return BR_BAD_ARG;
     dim3 grid((unsigned)((size_t)T * top), (F + 15) / 16);
     const size_t lds = (size_t)W * sizeof(float);
     const bool vec = W % (is_bf16 ? 8 : 4) == 0;
-#define RX_UP(TT, V) experts_up_kernel<TT, V><<<grid, 256, lds, s>>>((const TT*)h, (const TT*)w_gu, chosen, (TT*)y, W, F, top)
+#define RX_UP(TT, V) experts_up_kernel<TT, V><<<grid, 256, lds, s>>>((const TT*)h, (const TT*)w_gu, chosen, (TT*)y, W, F, top, E, limit, alpha)
     if (is_bf16) { if (vec) RX_UP(bf16, true); else RX_UP(bf16, false); }
     else { if (vec) RX_UP(float, true); else RX_UP(float, false); }
 #undef RX_UP
     return br_check_launch();
 }
 
-extern "C" int br_experts_down(const void* y, const void* w_down, const int* chosen, const float* share, float* x, int is_bf16,
-                               int T, int W, int F, int top, hipStream_t s) {
+// `h`: the input rows, which identity experts return (numbers from E on; null where there are none); `store`: x is
+// overwritten instead of added to.
+extern "C" int br_experts_down(const void* y, const void* w_down, const int* chosen, const float* share, const void* h, float* x,
+                               int is_bf16, int T, int W, int F, int top, int E, int store, hipStream_t s) {
     if (T <= 0) return BR_OK;
     if (W <= 0 || F <= 0 || top <= 0 || (size_t)top * F * 4 > 65536 || (W + 15) / 16 > 65535) return BR_BAD_ARG;
     dim3 grid(T, (W + 15) / 16);
     const size_t lds = (size_t)top * F * sizeof(float);
     const bool vec = F % (is_bf16 ? 8 : 4) == 0;
-#define RX_DOWN(TT, V) experts_down_kernel<TT, V><<<grid, 256, lds, s>>>((const TT*)y, (const TT*)w_down, chosen, share, x, W, F, top)
+#define RX_DOWN(TT, V) experts_down_kernel<TT, V><<<grid, 256, lds, s>>>((const TT*)y, (const TT*)w_down, chosen, share, (const TT*)h, x, W, F, top, E, store)
     if (is_bf16) { if (vec) RX_DOWN(bf16, true); else RX_DOWN(bf16, false); }
     else { if (vec) RX_DOWN(float, true); else RX_DOWN(float, false); }
 #undef RX_DOWN
@@ -366,14 +422,15 @@ extern "C" int br_experts_down(const void* y, const void* w_down, const int* cho
 // The (token, slot) pairs grouped by expert: first[e] .. first[e + 1] - 1 are the places of expert e's pairs in
 // `order` (pair numbers t * top + s), and place[pair] is where a pair went.  One workgroup: counts in LDS, a scan by
 // one thread, places handed out by counters.  Which of an expert's pairs comes first is left to the counters; a
-// pair's output does not depend on its place.
+// pair's output does not depend on its place.  Numbers from E - 1 on count as E - 1: with identity experts E is one more
+// than the experts with matrices, and the last bin holds the identities' pairs.
 __global__ __launch_bounds__(1024) void experts_sort_kernel(const int* __restrict__ chosen, int* __restrict__ first,
                                                             int* __restrict__ order, int* __restrict__ place, int n, int E) {
     extern __shared__ int cnt[];                   // [E] counts, then [E] counters
     int* cur = cnt + E;
     for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
     __syncthreads();
-    for (int i = threadIdx.x; i < n; i += 1024) atomicAdd(&cnt[chosen[i]], 1);
+    for (int i = threadIdx.x; i < n; i += 1024) atomicAdd(&cnt[min(chosen[i], E - 1)], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int at = 0;
@@ -382,7 +439,7 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int* __restric
     }
     __syncthreads();
     for (int i = threadIdx.x; i < n; i += 1024) {
-        const int p = atomicAdd(&cur[chosen[i]], 1);
+        const int p = atomicAdd(&cur[min(chosen[i], E - 1)], 1);
         order[p] = i;
         place[i] = p;
     }
@@ -395,40 +452,78 @@ extern "C" int br_experts_sort(const int* chosen, int* first, int* order, int* p
     return br_check_launch();
 }
 
-// rows[p, :] = h[order[p] / top, :]: the tokens' rows in the experts' order.  grid (pairs), 256 threads.
-template <typename T>
+// rows[p, :] = h[order[p] / top, :]: the tokens' rows in the experts' order, for the pairs before *n_rows (null: all; the
+// pairs of identity experts lie behind and need no copy).  grid (pairs), 256 threads; VEC: 16-byte loads.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void experts_gather_kernel(const T* __restrict__ h, const int* __restrict__ order,
-                                                             T* __restrict__ rows, int W, int top) {
+                                                             const int* __restrict__ n_rows, T* __restrict__ rows, int W, int top) {
+    if (n_rows && (int)blockIdx.x >= *n_rows) return;
     const T* src = h + (size_t)(order[blockIdx.x] / top) * W;
     T* dst = rows + (size_t)blockIdx.x * W;
-    for (int i = threadIdx.x; i < W; i += 256) dst[i] = src[i];
+    if (VEC) {
+        typedef typename rx_vec<T>::type vec_t;
+        for (int i = threadIdx.x; i < W / rx_vec<T>::N; i += 256) ((vec_t*)dst)[i] = ((const vec_t*)src)[i];
+    } else
+        for (int i = threadIdx.x; i < W; i += 256) dst[i] = src[i];
 }
 
-extern "C" int br_experts_gather(const void* h, const int* order, void* rows, int is_bf16, int n, int W, int top, hipStream_t s) {
+extern "C" int br_experts_gather(const void* h, const int* order, const int* n_rows, void* rows, int is_bf16, int n, int W, int top,
+                                 hipStream_t s) {
     if (n <= 0) return BR_OK;
     if (W <= 0 || top <= 0) return BR_BAD_ARG;
-    if (is_bf16) experts_gather_kernel<bf16><<<n, 256, 0, s>>>((const bf16*)h, order, (bf16*)rows, W, top);
-    else experts_gather_kernel<float><<<n, 256, 0, s>>>((const float*)h, order, (float*)rows, W, top);
+    const bool vec = W % (is_bf16 ? 8 : 4) == 0 && (((uintptr_t)h | (uintptr_t)rows) & 15) == 0;
+#define RX_GATHER(TT, V) experts_gather_kernel<TT, V><<<n, 256, 0, s>>>((const TT*)h, order, n_rows, (TT*)rows, W, top)
+    if (is_bf16) { if (vec) RX_GATHER(bf16, true); else RX_GATHER(bf16, false); }
+    else { if (vec) RX_GATHER(float, true); else RX_GATHER(float, false); }
+#undef RX_GATHER
     return br_check_launch();
 }
 
 // x[t, :] += sum_s share[t, s] * out[place[t * top + s], :] with out the experts' float outputs in their order;
-// slots in slot order.  grid (T, ceil(W / 256)).
+// slots in slot order.  With `chosen` (null: no identity experts) a slot whose expert number is E or more takes the
+// token's input row h[t, :] instead of an output.  `store`: x is overwritten instead of added to.
+// grid (T, ceil(W / (256 VEC))); VEC 4: four elements a thread (W in steps of 4, aligned).
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ out, const int* __restrict__ place,
-                                                              const float* __restrict__ share, float* __restrict__ x, int W, int top) {
-    const int t = blockIdx.x, i = blockIdx.y * 256 + threadIdx.x;
+                                                              const float* __restrict__ share, const int* __restrict__ chosen,
+                                                              const T* __restrict__ h, float* __restrict__ x, int W, int top, int E,
+                                                              int store) {
+    const int t = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * VEC;
     if (i >= W) return;
-    float sum = 0.f;
-    for (int s = 0; s < top; ++s)
-        sum = fmaf(share[(size_t)t * top + s], out[(size_t)place[(size_t)t * top + s] * W + i], sum);
-    x[(size_t)t * W + i] += sum;
+    float sum[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) sum[e] = 0.f;
+    for (int s = 0; s < top; ++s) {
+        const size_t pair = (size_t)t * top + s;
+        const float w = share[pair];
+        if (chosen && chosen[pair] >= E) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) sum[e] = fmaf(w, to_f32<T>(h[(size_t)t * W + i + e]), sum[e]);
+        } else {
+            const float* o = out + (size_t)place[pair] * W + i;
+            if (VEC == 4) {
+                const f32x4 v = *(const f32x4*)o;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) sum[e] = fmaf(w, v[e], sum[e]);
+            } else sum[0] = fmaf(w, o[0], sum[0]);
+        }
+    }
+    float* xr = x + (size_t)t * W + i;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) xr[e] = store ? sum[e] : xr[e] + sum[e];
 }
 
-extern "C" int br_experts_combine(const float* out, const int* place, const float* share, float* x, int T, int W, int top,
-                                  hipStream_t s) {
+extern "C" int br_experts_combine(const float* out, const int* place, const float* share, const int* chosen, const void* h,
+                                  int h_is_bf16, float* x, int T, int W, int top, int E, int store, hipStream_t s) {
     if (T <= 0) return BR_OK;
-    if (W <= 0 || top <= 0 || (W + 255) / 256 > 65535) return BR_BAD_ARG;
-    experts_combine_kernel<<<dim3(T, (W + 255) / 256), 256, 0, s>>>(out, place, share, x, W, top);
+    if (W <= 0 || top <= 0 || (W + 255) / 256 > 65535 || (chosen && !h)) return BR_BAD_ARG;
+    const bool vec = W % 4 == 0 && (((uintptr_t)out | (uintptr_t)x) & 15) == 0;
+    const int per = vec ? 1024 : 256;
+    const dim3 grid(T, (W + per - 1) / per);
+#define RX_COMBINE(TT, V) experts_combine_kernel<TT, V><<<grid, 256, 0, s>>>(out, place, share, chosen, (const TT*)h, x, W, top, E, store)
+    if (h_is_bf16) { if (vec) RX_COMBINE(bf16, 4); else RX_COMBINE(bf16, 1); }
+    else { if (vec) RX_COMBINE(float, 4); else RX_COMBINE(float, 1); }
+#undef RX_COMBINE
     return br_check_launch();
 }
 
@@ -441,10 +536,10 @@ extern "C" int br_experts_combine(const float* out, const int* place, const floa
 // order.  Experts without pairs cost a workgroup a load and a compare.
 //
 // `up`: rows of h gathered through `order` (pair -> token = pair / top), gate and up rows of the same f in the same
-// lane, y[p, f] = silu(g) * u in the experts' order.  grid (E, ceil(F / 32)).
+// lane, y[p, f] = silu(g) * u (or the clamped unit) in the experts' order.  grid (E, ceil(F / 32)).
 __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __restrict__ h, const bf16* __restrict__ w_gu,
                                                                  const int* __restrict__ first, const int* __restrict__ order,
-                                                                 bf16* __restrict__ y, int W, int F, int top) {
+                                                                 bf16* __restrict__ y, int W, int F, int top, float limit, float alpha) {
     __shared__ float red[3][2][16][64];
     const int e = blockIdx.x, f0 = blockIdx.y * 32;
     const int p0 = first[e], p1 = first[e + 1];
@@ -483,7 +578,7 @@ __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __r
                 const float gs = ((ag[r] + red[0][0][r][lane]) + red[1][0][r][lane]) + red[2][0][r][lane];
                 const float us = ((au[r] + red[0][1][r][lane]) + red[1][1][r][lane]) + red[2][1][r][lane];
                 const int ff = f0 + 8 * (r >> 2) + 4 * g + (r & 3);
-                if (ff < F) y[(size_t)p * F + ff] = (bf16)(gs / (1.0f + expf(-gs)) * us);
+                if (ff < F) y[(size_t)p * F + ff] = (bf16)rx_glu(gs, us, limit, alpha);
             }
         }
         __syncthreads();
@@ -539,9 +634,9 @@ __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* _
 extern "C" int br_experts_grouped_takes(int W, int F) { return W > 0 && F > 0 && W % 8 == 0 && F % 8 == 0; }
 
 extern "C" int br_experts_up_grouped(const void* h, const void* w_gu, const int* first, const int* order, void* y, int E,
-                                     int W, int F, int top, hipStream_t s) {
+                                     int W, int F, int top, float limit, float alpha, hipStream_t s) {
     if (!br_experts_grouped_takes(W, F) || E <= 0 || top <= 0 || (F + 31) / 32 > 65535) return BR_BAD_ARG;
-    experts_up_grouped_kernel<<<dim3(E, (F + 31) / 32), 256, 0, s>>>((const bf16*)h, (const bf16*)w_gu, first, order, (bf16*)y, W, F, top);
+    experts_up_grouped_kernel<<<dim3(E, (F + 31) / 32), 256, 0, s>>>((const bf16*)h, (const bf16*)w_gu, first, order, (bf16*)y, W, F, top, limit, alpha);
     return br_check_launch();
 }
 

@@ -86,10 +86,14 @@ class DecoderModel:
         self.final_norm = build_part("norm", spec.final_norm)
         self.lm_head = build_part("lm_head", spec.lm_head)
         self.positions = {name: build_part("position", ps) for name, ps in spec.positions.items()}
+        self.input_joins = {name: build_part("input_join", js) for name, js in spec.input_joins.items()}
         self.schedule = list(spec.schedule)
         for e in self.schedule:
             if not 0 <= e.layer < len(self.layers):
                 raise ConfigError(f"schedule names layer {e.layer}, the model has {len(self.layers)}")
+            if e.input_join is not None and e.input_join not in self.input_joins:
+                raise ConfigError(f"schedule entry of layer {e.layer} names the input join {e.input_join!r}, the model has "
+                                  f"{sorted(self.input_joins)}")
         written = set()
         for e in self.schedule:
             if e.cache is not None and self.layers[e.layer].mixer is not None:
@@ -141,6 +145,8 @@ class DecoderModel:
         yield self.lm_head, s.lm_head_prefix
         for name, p in self.positions.items():
             yield p, s.position_prefixes.get(name, f"position.{name}.")
+        for name, p in self.input_joins.items():
+            yield p, s.input_join_prefixes.get(name, f"join.{name}.")
 
     def weight_specs(self) -> List[TensorSpec]:
         out: List[TensorSpec] = []
@@ -247,6 +253,8 @@ class DecoderModel:
             # entries that add the embedding output again read a copy: the rows themselves move on
             x0 = ws.get("embedding_out", (T, H), torch.float32)
             x0.copy_(x)
+        for join in self.input_joins.values():
+            join.begin(x, step)
         step.prepared_norm = None
         for i, e in enumerate(self.schedule):
             layer = self.layers[e.layer]
@@ -254,10 +262,13 @@ class DecoderModel:
             if e.adds_embedding:
                 K.residual_add(x, x0)
                 step.prepared_norm = None          # what a product prepared for the next norm is of the rows before the sum
+            if e.input_join is not None:
+                self.input_joins[e.input_join].forward(x, step)
+                step.prepared_norm = None
             # the norm that reads the residual rows after this layer: the next scheduled layer's first
             # (the final norm reads chosen rows only and is left alone)
             step.norm_after_layer = None
-            if i + 1 < len(self.schedule):
+            if i + 1 < len(self.schedule) and self.schedule[i + 1].input_join is None:
                 step.norm_after_layer = self.layers[self.schedule[i + 1].layer].first_norm()
             ctx = (self._mixer_context(cache, e, i, None) if layer.mixer is not None
                    else MixerContext(unit=e.cache, writes_cache=e.writes_cache))

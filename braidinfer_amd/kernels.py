@@ -110,11 +110,12 @@ def rmsnorm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, eps: float,
 
 
 def layernorm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, eps: float, rows: Optional[torch.Tensor] = None,
-              center: bool = True, add: bool = False, then=None) -> None:
+              center: bool = True, add: bool = False, then=None, plain: bool = False) -> None:
     """out = norm(x) * w, or out += norm(x) * w with `add` (float `out`); `center` False: the RMS norm.
     `then` = (w2, out2, eps2, center2), with `add` only: the rows just added to are normed once more,
     out2 = norm2(out) * w2, in the same kernel; with w2 None out2 takes the rows just added to as they are, in its
-    own dtype (for a reader that takes the rows without a norm)."""
+    own dtype (for a reader that takes the rows without a norm).  `plain`: no norm at all, out = x * w or out += x * w
+    (with `center` False)."""
     _dev("layernorm", x, w, out, rows)
     H = x.shape[-1]
     R = out.shape[0]
@@ -134,11 +135,22 @@ def layernorm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, eps: float, r
         _req(add and (w2 is None or (w2.dtype == torch.float32 and w2.numel() == H)) and out2.shape == (R, H)
              and out2.data_ptr() not in (x.data_ptr(), out.data_ptr()), "layernorm: the second norm takes float weights [H] "
              "and rows [R, H] of their own, behind an add")
-    f = _fn("elementwise", "br_layernorm", [_P, _P, _P, c_int, _P, c_int, c_int, c_float, c_int, c_int, _P, _P, c_int,
+    _req(not (plain and center), "layernorm: rows that are only scaled are not centred")
+    f = _fn("elementwise", "br_layernorm", [_P, _P, _P, c_int, _P, c_int, c_int, c_float, c_int, c_int, c_int, _P, _P, c_int,
                                             c_float, c_int, _P])
     _check(f(_ptr(x), _ptr(w), _ptr(out), _is_bf16(out, "layernorm"), _ptr(rows), R, H, float(eps), int(center),
-             int(add), _ptr(w2), _ptr(out2), _is_bf16(out2, "layernorm") if out2 is not None else 0, float(eps2),
+             int(add), int(plain), _ptr(w2), _ptr(out2), _is_bf16(out2, "layernorm") if out2 is not None else 0, float(eps2),
              int(center2), _stream()), "layernorm")
+
+
+def rows_into(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = x in out's dtype: x float [T, H] dense, out [T, H] with dense rows that may lie further apart (a range of
+    columns of wider rows)."""
+    _dev("rows_into", x)
+    T, H = x.shape
+    _req(x.dtype == torch.float32 and out.is_cuda and out.shape == (T, H) and out.stride(1) == 1, "rows_into: x float32 [T, H], out [T, H] with dense rows")
+    f = _fn("elementwise", "br_rows_into", [_P, _P, c_int, c_int, c_int, c_size_t, _P])
+    _check(f(_ptr(x), _ptr(out), _is_bf16(out, "rows_into"), T, H, out.stride(0) if T > 1 else H, _stream()), "rows_into")
 
 
 def scale_(x: torch.Tensor, scale: float) -> None:
@@ -542,7 +554,8 @@ def pwa_prepare(qkv: torch.Tensor, bias: Optional[torch.Tensor], q_norm: Optiona
                 block_table: torch.Tensor, q_out: torch.Tensor, unit: torch.Tensor, v_first: Optional[torch.Tensor],
                 mix: Optional[torch.Tensor], v_role: int, nq: int, nkv: int, dk: int, dv: int, page: int,
                 write_cache: bool, values_from_keys: bool = False, q_temp_coef: float = 0.0, q_temp_every: int = 0,
-                maps: int = 1, row_ss: Optional[torch.Tensor] = None, pad_queries: bool = True) -> None:
+                maps: int = 1, row_ss: Optional[torch.Tensor] = None, pad_queries: bool = True, adjacent: bool = False,
+                q_scale: Optional[torch.Tensor] = None, v_eps: Optional[float] = None) -> None:
     """Float projection sums [T, nq*dk + nkv*dk + nkv*dv (+ more columns that are not read)] -> queries (normed,
     rotated) in `q_out` and the tokens' keys (normed, rotated) and values in their cache pages.  `v_role` 1 leaves
     the values in `v_first`, 2 mixes them with it by the scalar `mix`.  `values_from_keys`: there are no value
@@ -553,9 +566,12 @@ def pwa_prepare(qkv: torch.Tensor, bias: Optional[torch.Tensor], q_norm: Optiona
     zeros where the other maps' keys lie (the attention kernels then take nq * maps query heads of maps * dk).  `row_ss`
     (float scratch [T, 2]): the norm runs over the token's whole query (key) projection instead of over a head, with
     weights for the whole projection (`q_norm` [nq * maps * dk], `k_norm` [nkv * maps * dk]).  `pad_queries` False: the
-    rows of `q_out` are dk wide, without the zeros (for a kernel that takes `maps` itself)."""
+    rows of `q_out` are dk wide, without the zeros (for a kernel that takes `maps` itself).  `adjacent`: the rotation's
+    pairs are neighbouring elements instead of (i, i + rotary_dim/2).  `q_scale` float [nq]: a factor per query head on its
+    queries.  `v_eps`: every head's values are divided by their root mean square, sqrt(mean + v_eps), before they are stored
+    (not with `v_role`)."""
     _dev("pwa_prepare", qkv, bias, q_norm, k_norm, cos, sin, positions, seq_of_token, slots, block_table, q_out, unit,
-         v_first, mix, row_ss)
+         v_first, mix, row_ss, q_scale)
     T = qkv.shape[0]
     _req(maps >= 1 and (maps == 1 or not values_from_keys), "pwa_prepare: one or more maps; keys that serve as values have one")
     nqs, nks, kw = nq * maps, nkv * maps, maps * dk
@@ -571,6 +587,8 @@ def pwa_prepare(qkv: torch.Tensor, bias: Optional[torch.Tensor], q_norm: Optiona
              "pwa_prepare: norm weights float32 [dk], or of the whole projection with a norm over it")
     _req(not whole or (row_ss.dtype == torch.float32 and row_ss.numel() >= 2 * T and q_norm is not None and k_norm is not None),
          "pwa_prepare: a norm over the whole projection takes float scratch [T, 2] and weights for queries and keys")
+    _req(q_scale is None or (q_scale.dtype == torch.float32 and q_scale.numel() == nq), "pwa_prepare: q_scale float32 [query heads]")
+    _req(v_eps is None or (v_eps >= 0 and not v_role), "pwa_prepare: the values' norm takes an eps >= 0 and no mixing")
     _req(positions.numel() >= T and seq_of_token.numel() >= T, "pwa_prepare: positions shorter than tokens")
     _req(block_table.dim() == 2 and block_table.dtype == torch.int32, "pwa_prepare: block table int32 [slots, pages]")
     _req(q_out.shape == (T, nqs * (kw if pad_queries else dk)) and q_out.dtype == unit.dtype,
@@ -584,12 +602,13 @@ def pwa_prepare(qkv: torch.Tensor, bias: Optional[torch.Tensor], q_norm: Optiona
              "pwa_prepare: v_first float32 [T, nkv*dv]")
         _req(v_role != 2 or (mix is not None and mix.dtype == torch.float32 and mix.numel() == 1), "pwa_prepare: mix is one float")
     f = _fn("pooled_attention", "br_pwa_prepare",
-            [_P, _P, _P, _P, c_float, _P, _P, c_int, _P, _P, _P, _P, c_int, _P, _P, c_int, _P, _P] + [c_int] * 10 + [c_float, c_int, c_int, _P, c_int, c_int, _P])
+            [_P, _P, _P, _P, c_float, _P, _P, c_int, _P, _P, _P, _P, c_int, _P, _P, c_int, _P, _P] + [c_int] * 10 + [c_float, c_int, c_int, _P, c_int, c_int, c_int, _P, c_float, _P])
     _check(f(_ptr(qkv), _ptr(bias), _ptr(q_norm), _ptr(k_norm), float(eps), _ptr(cos), _ptr(sin), int(rotary_dim),
              _ptr(positions), _ptr(seq_of_token), _ptr(slots), _ptr(block_table), block_table.shape[1], _ptr(q_out),
              _ptr(unit), _is_bf16(unit, "pwa_prepare"), _ptr(v_first), _ptr(mix), int(v_role), T, nq, nkv, dk, dv, page,
              int(write_cache), int(qkv.shape[1]), int(bool(values_from_keys)), float(q_temp_coef), int(q_temp_every),
-             int(maps), _ptr(row_ss), dk if whole else 0, int(bool(pad_queries)), _stream()), "pwa_prepare")
+             int(maps), _ptr(row_ss), dk if whole else 0, int(bool(pad_queries)), int(bool(adjacent)),
+             _ptr(q_scale), -1.0 if v_eps is None else float(v_eps), _stream()), "pwa_prepare")
 
 
 def pwa_pair_combine(a: torch.Tensor, out: torch.Tensor, nq: int, dv: int, factor: float, eps: Optional[float],
@@ -1026,10 +1045,11 @@ def latent_prepare(q: torch.Tensor, dkv: Optional[torch.Tensor], c_weight: Optio
                    cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], rot: int, positions: torch.Tensor,
                    seq_of_token: torch.Tensor, slots: torch.Tensor, block_table: Optional[torch.Tensor],
                    cache: Optional[torch.Tensor], q_plain: torch.Tensor, q_wide: torch.Tensor, H: int, D: int, DR: int, R: int,
-                   page: int) -> None:
+                   page: int, halves: bool = False) -> None:
     """q float [T, H*(D+DR)] and dkv float [T, R+DR] (views whose rows may be strided; dkv None: nothing is kept):
     the normed latent and the rotated shared key part into the token's cache row, the queries' plain parts into
-    q_plain [T, H*D] and their rotated parts into q_wide [T, H*(R+DR)] behind each head's first R elements."""
+    q_plain [T, H*D] and their rotated parts into q_wide [T, H*(R+DR)] behind each head's first R elements.  The first
+    `rot` elements of a rotated part turn in pairs of neighbours, or with `halves` in pairs (i, i + rot/2)."""
     _dev("latent_prepare", c_weight, cos, sin, positions, seq_of_token, slots, block_table, cache, q_plain, q_wide)
     T = q.shape[0]
     _req(q.is_cuda and q.dtype == torch.float32 and q.shape == (T, H * (D + DR)) and q.stride(1) == 1, "latent_prepare: q float32 [T, H*(D+DR)]")
@@ -1045,24 +1065,28 @@ def latent_prepare(q: torch.Tensor, dkv: Optional[torch.Tensor], c_weight: Optio
         _req(block_table is not None and block_table.dim() == 2 and block_table.dtype == torch.int32, "latent_prepare: block table int32 [slots, pages]")
         ds = dkv.stride(0) if T > 1 else R + DR
     f = _fn("latent_attention", "br_latent_prepare",
-            [_P, c_size_t, _P, c_size_t, _P, c_float, _P, _P, _P, _P, _P, _P, c_int, _P, _P, _P] + [c_int] * 8 + [_P])
+            [_P, c_size_t, _P, c_size_t, _P, c_float, _P, _P, _P, _P, _P, _P, c_int, _P, _P, _P] + [c_int] * 9 + [_P])
     _check(f(_ptr(q), q.stride(0) if T > 1 else H * (D + DR), _ptr(dkv), ds, _ptr(c_weight), float(eps), _ptr(cos), _ptr(sin),
              _ptr(positions), _ptr(seq_of_token), _ptr(slots), _ptr(block_table), block_table.shape[1] if block_table is not None else 0,
-             _ptr(cache), _ptr(q_plain), _ptr(q_wide), _is_bf16(q_plain, "latent_prepare"), T, H, D, DR, R, int(rot), page, _stream()),
+             _ptr(cache), _ptr(q_plain), _ptr(q_wide), _is_bf16(q_plain, "latent_prepare"), T, H, D, DR, R, int(rot), int(bool(halves)), page, _stream()),
            "latent_prepare")
 
 
-def head_linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
+def head_linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> None:
     """out[t, h, :] = w[h] a[t, h, :] for every head in one launch: a [T, H, K] and out [T, H, N] may be views of
-    wider rows (strides between tokens and heads, dense last dimension); w [H, N, K] dense."""
+    wider rows (strides between tokens and heads, dense last dimension); w [H, N, K] dense.  `gate`: a float view
+    [T, H * N] (rows may be strided); the sums are multiplied by its sigmoid before they are rounded."""
     _dev("head_linear", w)
     T, H, K = a.shape
     N = w.shape[1]
     _req(a.is_cuda and out.is_cuda and a.dtype == w.dtype == out.dtype, "head_linear: one type, on the device")
     _req(w.shape == (H, N, K) and out.shape == (T, H, N) and a.stride(2) == 1 and out.stride(2) == 1, "head_linear: a [T, H, K], w [H, N, K], out [T, H, N]")
     lda, ldo = (a.stride(0) if T > 1 else H * K), (out.stride(0) if T > 1 else H * N)
-    f = _fn("latent_attention", "br_head_linear", [_P, c_size_t, c_size_t, _P, _P, c_size_t, c_size_t] + [c_int] * 5 + [_P])
-    _check(f(_ptr(a), lda, a.stride(1) if H > 1 else K, _ptr(w), _ptr(out), ldo, out.stride(1) if H > 1 else N, _is_bf16(a, "head_linear"),
+    _req(gate is None or (gate.is_cuda and gate.dtype == torch.float32 and gate.shape == (T, H * N) and gate.stride(1) == 1),
+         "head_linear: gate float32 [T, H * N]")
+    gs = 0 if gate is None else (gate.stride(0) if T > 1 else H * N)
+    f = _fn("latent_attention", "br_head_linear", [_P, c_size_t, c_size_t, _P, _P, c_size_t, c_size_t, _P, c_size_t] + [c_int] * 5 + [_P])
+    _check(f(_ptr(a), lda, a.stride(1) if H > 1 else K, _ptr(w), _ptr(out), ldo, out.stride(1) if H > 1 else N, _ptr(gate), gs, _is_bf16(a, "head_linear"),
              T, H, N, K, _stream()), "head_linear")
 
 
@@ -1095,14 +1119,36 @@ def route_sigmoid(scores: torch.Tensor, correction: Optional[torch.Tensor], chos
     _req(0 < top <= min(E, 64) and E <= 512, f"route_sigmoid: {top} of {E} experts is outside the kernel's sizes (512 experts, 64 chosen)")
     _req(groups >= 1 and E % groups == 0 and (groups == 1 or (1 <= keep <= groups and keep * (E // groups) >= top)),
          f"route_sigmoid: {groups} runs of experts of which {keep} are kept cannot give {top} of {E} experts")
-    f = _fn("routed_experts", "br_route_sigmoid", [_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, _P])
-    _check(f(_ptr(scores), _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, int(groups), int(keep), float(out_scale),
+    f = _fn("routed_experts", "br_route_corrected", _ROUTE_ARGS)
+    _check(f(_ptr(scores), E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, int(groups), int(keep), 0, 1, float(out_scale),
              _stream()), "route_sigmoid")
 
 
-def experts_up(h: torch.Tensor, w_gu: torch.Tensor, chosen: torch.Tensor, y: torch.Tensor) -> None:
+_ROUTE_ARGS = [_P, c_int, _P, _P, _P] + [c_int] * 7 + [c_float, _P]
+
+
+def route_softmax(scores: torch.Tensor, correction: Optional[torch.Tensor], chosen: torch.Tensor, share: torch.Tensor, top: int,
+                  out_scale: float = 1.0) -> None:
+    """scores float [T, E] (rows may be strided): s = the softmax over a row; the `top` numbers with the largest
+    s + correction (ties to the lower one) into chosen int32 [T, top], their s as they are, times `out_scale`, into share
+    float [T, top]."""
+    _dev("route_softmax", correction, chosen, share)
+    T, E = scores.shape
+    _req(scores.is_cuda and scores.dtype == torch.float32 and scores.stride(1) == 1 and (T <= 1 or scores.stride(0) >= E),
+         "route_softmax: float32 scores with dense rows")
+    _req(correction is None or (correction.dtype == torch.float32 and correction.numel() == E), "route_softmax: correction float32 [E]")
+    _req(chosen.dtype == torch.int32 and chosen.shape == (T, top) and share.dtype == torch.float32 and share.shape == (T, top),
+         "route_softmax: chosen int32 and share float32 [T, top]")
+    _req(0 < top <= min(E, 64) and E <= 512, f"route_softmax: {top} of {E} is outside the kernel's sizes (512 outputs, 64 chosen)")
+    f = _fn("routed_experts", "br_route_corrected", _ROUTE_ARGS)
+    _check(f(_ptr(scores), scores.stride(0) if T > 1 else E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, 1, 1, 1, 0,
+             float(out_scale), _stream()), "route_softmax")
+
+
+def experts_up(h: torch.Tensor, w_gu: torch.Tensor, chosen: torch.Tensor, y: torch.Tensor, limit: float = 0.0, alpha: float = 0.0) -> None:
     """y[t, s] = silu(W_gate[e] h[t]) * (W_up[e] h[t]) with e = chosen[t, s]; w_gu [E, 2 F, W] holds an expert's gate
-    rows, then its up rows; y [T, top, F]."""
+    rows, then its up rows; y [T, top, F].  `alpha` > 0: the clamped unit g sigmoid(alpha g) (u + 1), g bounded by `limit`
+    from above and u on both sides.  Numbers from E on are identity experts, whose y is left alone."""
     _dev("experts_up", h, w_gu, chosen, y)
     T, W = h.shape
     E, F2, _ = w_gu.shape
@@ -1110,12 +1156,14 @@ def experts_up(h: torch.Tensor, w_gu: torch.Tensor, chosen: torch.Tensor, y: tor
     _req(F2 % 2 == 0 and w_gu.shape == (E, F2, W) and y.shape == (T, top, F2 // 2) and chosen.shape == (T, top) and chosen.dtype == torch.int32, "experts_up: shapes")
     _req(h.dtype == w_gu.dtype == y.dtype, "experts_up: one type for rows and weights")
     _req(W <= 16384, "experts_up: rows wider than 16,384")
-    f = _fn("routed_experts", "br_experts_up", [_P, _P, _P, _P] + [c_int] * 5 + [_P])
-    _check(f(_ptr(h), _ptr(w_gu), _ptr(chosen), _ptr(y), _is_bf16(h, "experts_up"), T, W, F2 // 2, top, _stream()), "experts_up")
+    f = _fn("routed_experts", "br_experts_up", [_P, _P, _P, _P] + [c_int] * 6 + [c_float, c_float, _P])
+    _check(f(_ptr(h), _ptr(w_gu), _ptr(chosen), _ptr(y), _is_bf16(h, "experts_up"), T, W, F2 // 2, top, E, float(limit),
+             float(alpha), _stream()), "experts_up")
 
 
 def experts_sort(chosen: torch.Tensor, first: torch.Tensor, order: torch.Tensor, place: torch.Tensor, E: int) -> None:
-    """The (token, slot) pairs of chosen [T, top] grouped by expert: first int32 [E + 1], order and place int32 [T * top]."""
+    """The (token, slot) pairs of chosen [T, top] grouped by expert: first int32 [E + 1], order and place int32 [T * top].
+    Numbers from E - 1 on share the last bin (with identity experts, E is the experts with matrices and one more)."""
     _dev("experts_sort", chosen, first, order, place)
     n = chosen.numel()
     _req(chosen.dtype == first.dtype == order.dtype == place.dtype == torch.int32 and first.numel() == E + 1 and order.numel() == n
@@ -1124,36 +1172,48 @@ def experts_sort(chosen: torch.Tensor, first: torch.Tensor, order: torch.Tensor,
     _check(f(_ptr(chosen), _ptr(first), _ptr(order), _ptr(place), n, E, _stream()), "experts_sort")
 
 
-def experts_gather(h: torch.Tensor, order: torch.Tensor, rows: torch.Tensor, top: int) -> None:
-    """rows[p] = h[order[p] // top]."""
-    _dev("experts_gather", h, order, rows)
+def experts_gather(h: torch.Tensor, order: torch.Tensor, rows: torch.Tensor, top: int, n_rows: Optional[torch.Tensor] = None) -> None:
+    """rows[p] = h[order[p] // top], for p below the one int32 number in `n_rows` when it is given."""
+    _dev("experts_gather", h, order, rows, n_rows)
+    _req(n_rows is None or (n_rows.dtype == torch.int32 and n_rows.numel() == 1), "experts_gather: n_rows is one int32")
     n, W = rows.shape
     _req(h.dtype == rows.dtype and h.shape[1] == W and order.dtype == torch.int32 and order.numel() == n, "experts_gather: shapes")
-    f = _fn("routed_experts", "br_experts_gather", [_P, _P, _P, c_int, c_int, c_int, c_int, _P])
-    _check(f(_ptr(h), _ptr(order), _ptr(rows), _is_bf16(h, "experts_gather"), n, W, top, _stream()), "experts_gather")
+    f = _fn("routed_experts", "br_experts_gather", [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P])
+    _check(f(_ptr(h), _ptr(order), _ptr(n_rows), _ptr(rows), _is_bf16(h, "experts_gather"), n, W, top, _stream()), "experts_gather")
 
 
-def experts_combine(out: torch.Tensor, place: torch.Tensor, share: torch.Tensor, x: torch.Tensor) -> None:
-    """x[t] += sum_s share[t, s] * out[place[t * top + s]]; out float [T * top, W]."""
-    _dev("experts_combine", out, place, share, x)
+def experts_combine(out: torch.Tensor, place: torch.Tensor, share: torch.Tensor, x: torch.Tensor,
+                    chosen: Optional[torch.Tensor] = None, h: Optional[torch.Tensor] = None, experts: int = 0,
+                    store: bool = False) -> None:
+    """x[t] += sum_s share[t, s] * out[place[t * top + s]] (`store`: = instead of +=); out float [T * top, W].  With `chosen`
+    [T, top] and `h` [T, W], a slot whose number is `experts` or more (an identity expert) takes h[t] instead of an output."""
+    _dev("experts_combine", out, place, share, x, chosen, h)
+    _req((chosen is None) == (h is None) and (chosen is None or (chosen.dtype == torch.int32 and chosen.shape == share.shape and h.shape == x.shape)),
+         "experts_combine: chosen int32 [T, top] and h [T, W] come together")
     T, top = share.shape
     W = x.shape[1]
     _req(out.dtype == x.dtype == share.dtype == torch.float32 and place.dtype == torch.int32 and out.shape == (T * top, W)
          and x.shape == (T, W) and place.numel() == T * top, "experts_combine: shapes")
-    f = _fn("routed_experts", "br_experts_combine", [_P, _P, _P, _P, c_int, c_int, c_int, _P])
-    _check(f(_ptr(out), _ptr(place), _ptr(share), _ptr(x), T, W, top, _stream()), "experts_combine")
+    f = _fn("routed_experts", "br_experts_combine", [_P, _P, _P, _P, _P, c_int, _P] + [c_int] * 5 + [_P])
+    _check(f(_ptr(out), _ptr(place), _ptr(share), _ptr(chosen), _ptr(h), 0 if h is None else _is_bf16(h, "experts_combine"), _ptr(x),
+             T, W, top, int(experts), int(store), _stream()), "experts_combine")
 
 
-def experts_down(y: torch.Tensor, w_down: torch.Tensor, chosen: torch.Tensor, share: torch.Tensor, x: torch.Tensor) -> None:
-    """x[t] += sum_s share[t, s] * W_down[chosen[t, s]] y[t, s]; w_down [E, W, F], x float [T, W]."""
-    _dev("experts_down", y, w_down, chosen, share, x)
+def experts_down(y: torch.Tensor, w_down: torch.Tensor, chosen: torch.Tensor, share: torch.Tensor, x: torch.Tensor,
+                 h: Optional[torch.Tensor] = None, store: bool = False) -> None:
+    """x[t] += sum_s share[t, s] * W_down[chosen[t, s]] y[t, s] (`store`: = instead of +=); w_down [E, W, F], x float [T, W].
+    Where numbers from E on occur (identity experts), `h` [T, W] holds the rows they return."""
+    _dev("experts_down", y, w_down, chosen, share, x, h)
+    _req(h is None or (h.shape == x.shape and h.dtype == y.dtype), "experts_down: h [T, W] of y's type")
     T, top, F = y.shape
     E, W, _ = w_down.shape
     _req(w_down.shape == (E, W, F) and x.shape == (T, W) and x.dtype == torch.float32 and chosen.shape == (T, top) and share.shape == (T, top), "experts_down: shapes")
     _req(y.dtype == w_down.dtype and chosen.dtype == torch.int32 and share.dtype == torch.float32, "experts_down: types")
     _req(top * F <= 16384, "experts_down: more than 16,384 inner elements a token")
-    f = _fn("routed_experts", "br_experts_down", [_P, _P, _P, _P, _P] + [c_int] * 5 + [_P])
-    _check(f(_ptr(y), _ptr(w_down), _ptr(chosen), _ptr(share), _ptr(x), _is_bf16(y, "experts_down"), T, W, F, top, _stream()), "experts_down")
+    f = _fn("routed_experts", "br_experts_down", [_P, _P, _P, _P, _P, _P] + [c_int] * 7 + [_P])
+    # without identity experts every number is below E
+    _check(f(_ptr(y), _ptr(w_down), _ptr(chosen), _ptr(share), _ptr(h), _ptr(x), _is_bf16(y, "experts_down"), T, W, F, top,
+             E if h is not None else 1 << 30, int(store), _stream()), "experts_down")
 
 
 def experts_grouped_takes(dtype: torch.dtype, W: int, F: int) -> bool:
@@ -1161,18 +1221,20 @@ def experts_grouped_takes(dtype: torch.dtype, W: int, F: int) -> bool:
     return dtype == torch.bfloat16 and W % 8 == 0 and F % 8 == 0
 
 
-def experts_up_grouped(h: torch.Tensor, w_gu: torch.Tensor, first: torch.Tensor, order: torch.Tensor, y: torch.Tensor, top: int) -> None:
+def experts_up_grouped(h: torch.Tensor, w_gu: torch.Tensor, first: torch.Tensor, order: torch.Tensor, y: torch.Tensor, top: int,
+                       limit: float = 0.0, alpha: float = 0.0) -> None:
     """y[p] = silu(W_gate[e] h[t]) * (W_up[e] h[t]) for the pairs p of `experts_sort` (t = order[p] // top, e the
-    expert whose run holds p); y [pairs, F] in the experts' order."""
+    expert whose run holds p; `alpha` > 0: the clamped unit, as in `experts_up`); y [pairs, F] in the experts' order."""
     _dev("experts_up_grouped", h, w_gu, first, order, y)
     T, W = h.shape
     E, F2, _ = w_gu.shape
     n = order.numel()
     _req(experts_grouped_takes(h.dtype, W, F2 // 2) and w_gu.dtype == y.dtype == torch.bfloat16, "experts_up_grouped: bfloat16, widths in steps of 8")
-    _req(w_gu.shape == (E, F2, W) and y.shape == (n, F2 // 2) and first.numel() == E + 1 and n == T * top
+    _req(w_gu.shape == (E, F2, W) and y.shape == (n, F2 // 2) and first.numel() in (E + 1, E + 2) and n == T * top
          and first.dtype == order.dtype == torch.int32, "experts_up_grouped: shapes")
-    f = _fn("routed_experts", "br_experts_up_grouped", [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, _P])
-    _check(f(_ptr(h), _ptr(w_gu), _ptr(first), _ptr(order), _ptr(y), E, W, F2 // 2, top, _stream()), "experts_up_grouped")
+    f = _fn("routed_experts", "br_experts_up_grouped", [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_float, _P])
+    _check(f(_ptr(h), _ptr(w_gu), _ptr(first), _ptr(order), _ptr(y), E, W, F2 // 2, top, float(limit), float(alpha), _stream()),
+           "experts_up_grouped")
 
 
 def experts_down_grouped(y: torch.Tensor, w_down: torch.Tensor, first: torch.Tensor, out: torch.Tensor) -> None:
@@ -1181,7 +1243,7 @@ def experts_down_grouped(y: torch.Tensor, w_down: torch.Tensor, first: torch.Ten
     n, F = y.shape
     E, W, _ = w_down.shape
     _req(experts_grouped_takes(y.dtype, W, F) and w_down.dtype == torch.bfloat16 and out.dtype == torch.float32, "experts_down_grouped: types")
-    _req(w_down.shape == (E, W, F) and out.shape == (n, W) and first.numel() == E + 1 and first.dtype == torch.int32, "experts_down_grouped: shapes")
+    _req(w_down.shape == (E, W, F) and out.shape == (n, W) and first.numel() in (E + 1, E + 2) and first.dtype == torch.int32, "experts_down_grouped: shapes")
     f = _fn("routed_experts", "br_experts_down_grouped", [_P, _P, _P, _P, c_int, c_int, c_int, _P])
     _check(f(_ptr(y), _ptr(w_down), _ptr(first), _ptr(out), E, W, F, _stream()), "experts_down_grouped")
 
@@ -1193,21 +1255,25 @@ def experts_gemm(a: torch.Tensor, w: torch.Tensor, first: torch.Tensor, out: tor
     n, Kd = a.shape
     E, N, _ = w.shape
     _req(a.dtype == w.dtype == torch.bfloat16 and Kd % 8 == 0 and w.shape == (E, N, Kd) and out.shape == (n, N)
-         and first.dtype == torch.int32 and first.numel() == E + 1, "experts_gemm: bfloat16 [pairs, K] x [E, N, K], K in steps of 8")
+         and first.dtype == torch.int32 and first.numel() in (E + 1, E + 2), "experts_gemm: bfloat16 [pairs, K] x [E, N, K], K in steps of 8")
     f = _fn("routed_experts", "br_experts_gemm", [_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P])
     _check(f(_ptr(a), _ptr(w), _ptr(first), _ptr(out), _is_bf16(out, "experts_gemm"), n, E, N, Kd, _stream()), "experts_gemm")
 
 
 # ------------------------------------------------------------- clamped gated unit -----
-def clamped_glu(gu: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, limit: float, alpha: float) -> None:
-    """out = g sigmoid(alpha g) (u + 1), g = min(gate + b, limit), u = clamp(up + b, -limit, limit), from the float sums
-    gu [T, 2 I] (gate | up) and their biases [2 I]."""
+def clamped_glu(gu: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, limit: float, alpha: float,
+                row_gate: Optional[torch.Tensor] = None) -> None:
+    """out = g sigmoid(alpha g) (u + 1), g = min(gate + b, limit), u = clamp(up + b, -limit, limit), from gu [T, 2 I]
+    (gate | up; float sums, or bfloat16 with a bfloat16 `out`) and their biases [2 I].  `row_gate`: a float view [T]
+    (one number a row, any stride); the rows are multiplied by its sigmoid."""
     _dev("clamped_glu", gu, bias, out)
     T, I2 = gu.shape
-    _req(gu.dtype == torch.float32 and I2 % 2 == 0 and out.shape == (T, I2 // 2), "clamped_glu: gu float32 [T, 2 I], out [T, I]")
+    _req(I2 % 2 == 0 and out.shape == (T, I2 // 2) and (gu.dtype == torch.float32 or out.dtype == gu.dtype), "clamped_glu: gu [T, 2 I] float32 (or bfloat16 like out), out [T, I]")
     _req(bias is None or (bias.dtype == torch.float32 and bias.numel() == I2), "clamped_glu: bias float32 [2 I]")
-    f = _fn("elementwise", "br_clamped_glu", [_P, _P, _P, c_int, c_int, c_int, c_float, c_float, _P])
-    _check(f(_ptr(gu), _ptr(bias), _ptr(out), _is_bf16(out, "clamped_glu"), T, I2 // 2, float(limit), float(alpha), _stream()), "clamped_glu")
+    _req(row_gate is None or (row_gate.is_cuda and row_gate.dtype == torch.float32 and row_gate.shape == (T,)), "clamped_glu: row_gate float32 [T]")
+    f = _fn("elementwise", "br_clamped_glu", [_P, c_int, _P, _P, c_size_t, _P, c_int, c_int, c_int, c_float, c_float, _P])
+    _check(f(_ptr(gu), _is_bf16(gu, "clamped_glu"), _ptr(bias), _ptr(row_gate), 0 if row_gate is None else row_gate.stride(0), _ptr(out),
+             _is_bf16(out, "clamped_glu"), T, I2 // 2, float(limit), float(alpha), _stream()), "clamped_glu")
 
 
 def add_bias_rows(x: torch.Tensor, bias: torch.Tensor) -> None:

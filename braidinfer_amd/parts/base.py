@@ -10,6 +10,8 @@ configuration or name.  Kinds:
                      sequence: a `CacheNeed` (growing keys/values) and/or a `StateNeed`
                      (fixed size)
 * `FeedForward`      adds its output to the residual stream
+* `InputJoin`        rewrites the residual rows from themselves and the embedding output, between
+                     two entries of the run order
 * block arrangements functions that run one layer's parts in order
 
 Tensors: the residual stream `x` is float32 `[T, hidden]` in both precisions; `h` is the
@@ -75,6 +77,10 @@ class Part:
     # instead of the normed rows and a `ResidualSink` instead of the residual tensor, which
     # lets the product that adds into the stream prepare the norm that reads it next.
     through_linear_only = False
+    # A mixer or feed-forward that reads normed rows but can store its output instead of adding it sets this: where an
+    # arrangement wants a branch's own output, it is handed a `ResidualSink` with `overwrite` over rows that hold nothing
+    # yet (without it, rows of zeros).
+    stores_output = False
 
     def weight_specs(self, prefix: str) -> List[TensorSpec]:
         return []
@@ -228,6 +234,17 @@ class FeedForward(Part):
         raise NotImplementedError
 
 
+class InputJoin(Part):
+    """Runs in front of a run-order entry that names it (`ScheduleEntry.input_join`)."""
+
+    def begin(self, x: torch.Tensor, step) -> None:
+        """Called once a step with the embedding output, before the first entry: keep what `forward` needs of it."""
+
+    def forward(self, x: torch.Tensor, step) -> None:
+        """Rewrite the residual rows `x` in place."""
+        raise NotImplementedError
+
+
 class Embedding(Part):
     def forward(self, tokens: torch.Tensor, out: torch.Tensor) -> None:
         raise NotImplementedError
@@ -240,7 +257,7 @@ class OutputHead(Part):
 
 # ------------------------------------------------------------------ registries ------
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Any]]] = {
-    "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "embedding": {}, "lm_head": {}, "block": {},
+    "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "embedding": {}, "lm_head": {}, "input_join": {}, "block": {},
 }
 
 

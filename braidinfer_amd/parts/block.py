@@ -68,7 +68,8 @@ class SandwichResidual:
     "feed_forward", "feed_forward_out" (an absent one is left out).  The half writes its output
     into float rows of its own; the norm behind it adds the normed rows to the residual rows, so
     the sum is a float add in that kernel, and where it can it also leaves the norm that reads the
-    rows next (the other half's, or the next layer's first) in the same pass."""
+    rows next (the other half's, or the next layer's first) in the same pass.  What stands behind a half need not
+    norm: a `layer_scale` there gives x += s * part(norm_in(x))."""
 
     def first_norm(self, layer):
         return layer.norms.get("mixer") if layer.mixer is not None else layer.norms.get("feed_forward")
@@ -102,7 +103,7 @@ class SandwichResidual:
             part.forward(h, x, step, *extra)
             return
         y = step.ws.get("branch_out", tuple(x.shape), x.dtype)
-        if part.through_linear_only:
+        if part.through_linear_only or part.stores_output:
             part.forward(h, ResidualSink(y, None, overwrite=True), step, *extra)
         else:
             y.zero_()

@@ -12,7 +12,10 @@ checkpoints the reference loads; "" where the prefix is the whole name).
 
 `rows`: no norm at all, y = x in the compute dtype, for a half of a layer that reads the residual rows themselves
 (a design that norms a half's output only).  It has no weights; a norm that adds behind the half before can leave
-these rows in the same kernel, as it would leave a following norm's."""
+these rows in the same kernel, as it would leave a following norm's.
+
+`layer_scale`: no norm either, y = x * w channel by channel with a learnt vector: what stands behind a half whose output
+is scaled before it joins the residual rows."""
 from __future__ import annotations
 
 from typing import Dict, List, Optional
@@ -140,6 +143,34 @@ class PlainRows(Norm):
         return None, 0.0, False          # no weight: the kernel behind another norm leaves the rows as they are
 
 
+class LayerScale(Norm):
+    """Rows times a learnt vector, float."""
+
+    graph_safe = True
+
+    def __init__(self, size: int, tensor: str = "weight"):
+        self.size, self.tensor = int(size), tensor
+        self.weight: Optional[torch.Tensor] = None
+
+    def weight_specs(self, prefix: str) -> List[TensorSpec]:
+        return [TensorSpec(prefix + self.tensor, (self.size,), kind="vector", init="ones")]
+
+    def load(self, tensors: Dict[str, torch.Tensor], prefix: str, rt: Runtime) -> None:
+        self.rt = rt
+        self.weight = rt.own(tensors[prefix + self.tensor].to(torch.float32))
+
+    def forward(self, x, out, rows=None):
+        K.layernorm(x, self.weight, out, 0.0, rows, center=False, plain=True)
+        return out
+
+    def add_normed(self, y, x, then=None, then_out=None):
+        nxt = then.then_args() if then is not None and then_out is not None else None
+        K.layernorm(y, self.weight, x, 0.0, center=False, add=True, plain=True,
+                    then=(nxt[0], then_out, nxt[1], nxt[2]) if nxt else None)
+        return nxt is not None
+
+
+register_part("norm", "layer_scale", LayerScale, replace=True)
 register_part("norm", "rows", PlainRows, replace=True)
 register_part("norm", "rmsnorm", RMSNorm, replace=True)
 register_part("norm", "layernorm", LayerNorm, replace=True)

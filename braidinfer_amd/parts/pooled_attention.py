@@ -16,7 +16,9 @@ Further options, each a parameter: the values may be the keys as projected, befo
 no value matrix); the query/key norm may go without weights (`qk_norm_weights` False); the query may be multiplied
 by a temperature that grows with the logarithm of the position, 1 + c ln(floor((p + 1) / n) + 1) (`q_temp` = (c, n));
 the heads' outputs may pass a sigmoid gate projected from the mixer's input, one number per output element or one
-per head (`gate` "element" / "head"), before the output projection; `out_scale` multiplies what the mixer adds to the
+per head (`gate` "element" / "head"), before the output projection; a learnt factor per head may multiply its scores
+(`head_temp`: it rides on the queries); every head's value may be divided by its root mean square over the head, without
+a weight, before it is stored (`v_norm_eps`); the rotation's pairs are the encoding's, (i, i + dims/2) or neighbours; `out_scale` multiplies what the mixer adds to the
 residual rows (it rides on the gate, or on the output matrix where there is none).
 
 Further rules of what a query sees, each a parameter: `chunk` C cuts the sequence into runs of C positions counted
@@ -82,7 +84,7 @@ class PooledWindowAttention(Mixer):
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "gate": "g_proj.weight",
              "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
              "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "value_mix": "value_mix", "sink": "sink",
-             "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
+             "head_temp": "temp", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int, value_dim: int,
                  window: int, pool: int = 0, scale: Optional[float] = None, sink: bool = False, bias: bool = False,
@@ -91,7 +93,8 @@ class PooledWindowAttention(Mixer):
                  names: Optional[Dict[str, str]] = None, values_from_keys: bool = False, qk_norm_weights: bool = True,
                  q_temp=None, gate: Optional[str] = None, out_scale: float = 1.0, chunk: Optional[int] = None,
                  keep_first: int = 0, softcap: Optional[float] = None, qk_norm_over: str = "head", maps: int = 1,
-                 diff: Optional[float] = None, head_norm_eps: Optional[float] = None):
+                 diff: Optional[float] = None, head_norm_eps: Optional[float] = None, head_temp: bool = False,
+                 v_norm_eps: Optional[float] = None):
         """`qk_norm_eps` None: no query/key norm.  `value_mix`: None, "source" (this layer's values are what
         later layers of the same `value_mix_group` mix with; its own scalar is loaded and unused) or "mix"."""
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
@@ -118,6 +121,8 @@ class PooledWindowAttention(Mixer):
             raise ConfigError("attention: one map, or two with the constant `diff` (then without keys as values, gate or pooled blocks)")
         if int(maps) * key_dim > MAX_WIDTH:
             raise ConfigError(f"attention: {maps} maps of {key_dim} make key rows wider than {MAX_WIDTH}")
+        if v_norm_eps is not None and (not float(v_norm_eps) >= 0 or value_mix is not None or values_from_keys):
+            raise ConfigError("attention: a norm of the values takes an eps >= 0 and values of their own, without mixing")
         if sink not in (True, False, "learnt"):
             raise ConfigError(f"attention: sink is False, True (a score of 0) or 'learnt', got {sink!r}")
         self.H, self.nq, self.nkv = int(hidden_size), int(num_heads), int(num_kv_heads)
@@ -137,6 +142,9 @@ class PooledWindowAttention(Mixer):
         self.maps, self.diff = int(maps), (None if diff is None else float(diff))
         self.head_norm_eps = None if head_norm_eps is None else float(head_norm_eps)
         self.kw = self.maps * self.dk          # a key row of the cache, and a query row the kernels see
+        self.head_temp, self.temps = bool(head_temp), None
+        self.v_norm_eps = None if v_norm_eps is None else float(v_norm_eps)
+        self.adjacent = False                  # the encoding's pairs; set by check_positions
         self.sinks = None
         self.pair_factor = 0.0
         self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
@@ -168,6 +176,8 @@ class PooledWindowAttention(Mixer):
                     TensorSpec(prefix + n["k_norm"], (self.nkv * self.kw if whole else self.dk,), kind="vector", init="ones")]
         if self.maps == 2:
             out += [TensorSpec(prefix + n[x], (self.dk,), kind="vector", init="normal") for x in ("lq1", "lk1", "lq2", "lk2")]
+        if self.head_temp:
+            out.append(TensorSpec(prefix + n["head_temp"], (self.nq,), kind="vector", init="ones"))
         if self.learnt_sink:
             out.append(TensorSpec(prefix + n["sink"], (self.nq,), kind="vector", init="normal"))
         if self.value_mix is not None:
@@ -197,6 +207,8 @@ class PooledWindowAttention(Mixer):
             self.q_norm = self.k_norm = ones
         if self.value_mix == "mix":
             self.mix = rt.own(tensors[prefix + n["value_mix"]].to(torch.float32).reshape(1))
+        if self.head_temp:
+            self.temps = rt.own(tensors[prefix + n["head_temp"]].to(torch.float32).reshape(-1))
         if self.learnt_sink:
             self.sinks = rt.own(tensors[prefix + n["sink"]].to(torch.float32).reshape(-1))
             if self.maps == 2:          # both maps of a head carry the head's sink
@@ -227,9 +239,10 @@ class PooledWindowAttention(Mixer):
         if getattr(enc, "gives", None) not in ("rotary", "embedding", "none"):
             raise ConfigError(f"attention cannot use the position encoding {self.position!r}: it gives {getattr(enc, 'gives', None)!r}")
         self._expects_tables = enc.gives == "rotary"
-        if self._expects_tables and (enc.rotary_dim > self.dk or getattr(enc, "pairing", "half") != "half"):
+        if self._expects_tables and (enc.rotary_dim > self.dk or getattr(enc, "pairing", "half") not in ("half", "adjacent")):
             raise ConfigError(f"attention: the encoding {self.position!r} rotates {enc.rotary_dim} elements in "
-                              f"{getattr(enc, 'pairing', None)!r} pairs; this mixer takes up to {self.dk} in 'half' pairs")
+                              f"{getattr(enc, 'pairing', None)!r} pairs; this mixer takes up to {self.dk} in 'half' or 'adjacent' pairs")
+        self.adjacent = self._expects_tables and getattr(enc, "pairing", "half") == "adjacent"
 
     # ---- one step ----------------------------------------------------------------------
     def forward(self, h, x, step, ctx: MixerContext) -> None:
@@ -272,7 +285,7 @@ class PooledWindowAttention(Mixer):
                       step.positions, step.seq_of_token, step.slots, ctx.block_table, q, unit, v_first, self.mix, role,
                       nq, nkv, dk, dv, ctx.page_tokens, ctx.writes_cache, self.values_from_keys,
                       self.q_temp[0] if self.q_temp else 0.0, self.q_temp[1] if self.q_temp else 0, maps=maps, row_ss=row_ss,
-                      pad_queries=pad)
+                      pad_queries=pad, adjacent=self.adjacent, q_scale=self.temps, v_eps=self.v_norm_eps)
         nq, dk = nq * maps, (kw if pad else dk)
         mask = dict(chunk=self.chunk, keep=self.keep_first, softcap=self.softcap)
         pooled = ctx.others.get("pooled")
