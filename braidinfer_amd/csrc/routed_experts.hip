@@ -530,11 +530,47 @@ extern "C" int br_experts_combine(const float* out, const int* place, const floa
 // ------------------------------------------- few tokens, every expert read once -----
 // bfloat16 on the matrix cores, for steps whose pairs were grouped by `sort` on the device (nothing comes back to
 // the host, so the step can be recorded): a workgroup owns 32 output rows of one expert's matrix and walks that
-// expert's pairs 32 at a time, so an expert's weights are read once per 32 of its pairs instead of once per pair.
-// Its four waves share k (wave w takes the k-steps of 16 numbered w, w + 4, ...), v_mfma_f32_32x32x16_bf16 with
-// the weight rows as the first operand, both operands straight from memory; the waves' sums meet in LDS in wave
-// order.  Experts without pairs cost a workgroup a load and a compare.
-//
+// expert's pairs 64 at a time (as two tiles of 32, or one where no more are left), so an expert's weights are read once
+// per 64 of its pairs instead of once per pair.  Its four waves share k in runs of 64 (wave w takes the runs w, w + 4,
+// ...: the four loads a lane makes of a row's run fall into one line of 128 bytes, one after the other),
+// v_mfma_f32_32x32x16_bf16 with the weight rows as the first operand, both operands straight from memory; the waves'
+// sums meet in LDS in wave order.  Experts without pairs cost a workgroup a load and a compare.
+
+// acc[tile][matrix] += the run-of-64 share of this wave: NM weight rows `w` (one a matrix) against the pairs' rows `a`
+// of one or two tiles.  Rows of the operands beyond the matrix's or the expert's last give results that nobody reads;
+// elements beyond K are zeros.
+template <int NM, int NT>
+__device__ __forceinline__ void rx_walk(const bf16* const (&w)[NM], const bf16* const (&a)[NT], int K, int wave, int g,
+                                        f32x16 (&acc)[2][NM]) {
+    bf16x8 zero;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) zero[i] = (bf16)0.f;
+    for (int k0 = wave * 64; k0 < K; k0 += 256) {
+        bf16x8 wf[NM][4], af[NT][4];
+        const bool whole = k0 + 64 <= K;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int k = k0 + 16 * j + 8 * g;
+            const bool on = whole || k < K;
+            const int kk = on ? k : 0;
+#pragma unroll
+            for (int m = 0; m < NM; ++m) wf[m][j] = *(const bf16x8*)(w[m] + kk);
+#pragma unroll
+            for (int t = 0; t < NT; ++t) {
+                af[t][j] = *(const bf16x8*)(a[t] + kk);
+                if (!on) af[t][j] = zero;
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+#pragma unroll
+                for (int m = 0; m < NM; ++m)
+                    acc[t][m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[m][j], af[t][j], acc[t][m], 0, 0, 0);
+    }
+}
+
 // `up`: rows of h gathered through `order` (pair -> token = pair / top), gate and up rows of the same f in the same
 // lane, y[p, f] = silu(g) * u (or the clamped unit) in the experts' order.  grid (E, ceil(F / 32)).
 __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __restrict__ h, const bf16* __restrict__ w_gu,
@@ -548,40 +584,43 @@ __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __r
     const int c = lane & 31, g = lane >> 5;
     const int f = f0 + c;
     const bf16* wg = w_gu + ((size_t)e * 2 * F + (f < F ? f : F - 1)) * W;
-    const bf16* wu = wg + (size_t)F * W;
-    bf16x8 zero;
+    const bf16* const w[2] = {wg, wg + (size_t)F * W};
+    for (int pb = p0; pb < p1; pb += 64) {
+        const bool two = pb + 32 < p1;
+        f32x16 acc[2][2];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) zero[i] = (bf16)0.f;
-    for (int pb = p0; pb < p1; pb += 32) {
-        const int p = pb + c;
-        const bf16* arow = h + (size_t)(order[p < p1 ? p : p1 - 1] / top) * W;
-        f32x16 ag, au;
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) { ag[r] = 0.f; au[r] = 0.f; }
-        for (int k0 = wave * 16; k0 < W; k0 += 64) {
-            const int k = k0 + 8 * g;
-            const bool on = k < W;
-            const bf16x8 af = (on && p < p1) ? *(const bf16x8*)(arow + k) : zero;
-            const bf16x8 gf = (on && f < F) ? *(const bf16x8*)(wg + k) : zero;
-            const bf16x8 uf = (on && f < F) ? *(const bf16x8*)(wu + k) : zero;
-            ag = __builtin_amdgcn_mfma_f32_32x32x16_bf16(gf, af, ag, 0, 0, 0);
-            au = __builtin_amdgcn_mfma_f32_32x32x16_bf16(uf, af, au, 0, 0, 0);
+            for (int r = 0; r < 16; ++r) { acc[t][0][r] = 0.f; acc[t][1][r] = 0.f; }
+        const int pa = min(pb + c, p1 - 1), pz = min(pb + 32 + c, p1 - 1);
+        const bf16* a0 = h + (size_t)(order[pa] / top) * W;
+        if (two) {
+            const bf16* const a[2] = {a0, h + (size_t)(order[pz] / top) * W};
+            rx_walk<2, 2>(w, a, W, wave, g, acc);
+        } else {
+            const bf16* const a[1] = {a0};
+            rx_walk<2, 1>(w, a, W, wave, g, acc);
         }
-        if (wave > 0) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) { red[wave - 1][0][r][lane] = ag[r]; red[wave - 1][1][r][lane] = au[r]; }
-        }
-        __syncthreads();
-        if (wave == 0 && p < p1) {
+        for (int t = 0; t < 2; ++t) {
+            if (t == 1 && !two) break;
+            if (wave > 0) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) {
-                const float gs = ((ag[r] + red[0][0][r][lane]) + red[1][0][r][lane]) + red[2][0][r][lane];
-                const float us = ((au[r] + red[0][1][r][lane]) + red[1][1][r][lane]) + red[2][1][r][lane];
-                const int ff = f0 + 8 * (r >> 2) + 4 * g + (r & 3);
-                if (ff < F) y[(size_t)p * F + ff] = (bf16)rx_glu(gs, us, limit, alpha);
+                for (int r = 0; r < 16; ++r) { red[wave - 1][0][r][lane] = acc[t][0][r]; red[wave - 1][1][r][lane] = acc[t][1][r]; }
             }
+            __syncthreads();
+            const int p = pb + 32 * t + c;
+            if (wave == 0 && p < p1) {
+#pragma unroll
+                for (int r = 0; r < 16; ++r) {
+                    const float gs = ((acc[t][0][r] + red[0][0][r][lane]) + red[1][0][r][lane]) + red[2][0][r][lane];
+                    const float us = ((acc[t][1][r] + red[0][1][r][lane]) + red[1][1][r][lane]) + red[2][1][r][lane];
+                    const int ff = f0 + 8 * (r >> 2) + 4 * g + (r & 3);
+                    if (ff < F) y[(size_t)p * F + ff] = (bf16)rx_glu(gs, us, limit, alpha);
+                }
+            }
+            __syncthreads();
         }
-        __syncthreads();
     }
 }
 
@@ -597,36 +636,40 @@ __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* _
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int c = lane & 31, g = lane >> 5;
     const int n = n0 + c;
-    const bf16* wr = w_down + ((size_t)e * W + (n < W ? n : W - 1)) * F;
-    bf16x8 zero;
+    const bf16* const w[1] = {w_down + ((size_t)e * W + (n < W ? n : W - 1)) * F};
+    for (int pb = p0; pb < p1; pb += 64) {
+        const bool two = pb + 32 < p1;
+        f32x16 acc[2][1];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) zero[i] = (bf16)0.f;
-    for (int pb = p0; pb < p1; pb += 32) {
-        const int p = pb + c;
-        const bf16* arow = y + (size_t)(p < p1 ? p : p1 - 1) * F;
-        f32x16 acc;
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) acc[r] = 0.f;
-        for (int k0 = wave * 16; k0 < F; k0 += 64) {
-            const int k = k0 + 8 * g;
-            const bool on = k < F;
-            const bf16x8 af = (on && p < p1) ? *(const bf16x8*)(arow + k) : zero;
-            const bf16x8 wf = (on && n < W) ? *(const bf16x8*)(wr + k) : zero;
-            acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf, af, acc, 0, 0, 0);
+            for (int r = 0; r < 16; ++r) acc[t][0][r] = 0.f;
+        const bf16* a0 = y + (size_t)min(pb + c, p1 - 1) * F;
+        if (two) {
+            const bf16* const a[2] = {a0, y + (size_t)min(pb + 32 + c, p1 - 1) * F};
+            rx_walk<1, 2>(w, a, F, wave, g, acc);
+        } else {
+            const bf16* const a[1] = {a0};
+            rx_walk<1, 1>(w, a, F, wave, g, acc);
         }
-        if (wave > 0) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) red[wave - 1][r][lane] = acc[r];
-        }
-        __syncthreads();
-        if (wave == 0 && p < p1) {
+        for (int t = 0; t < 2; ++t) {
+            if (t == 1 && !two) break;
+            if (wave > 0) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) {
-                const int nn = n0 + 8 * (r >> 2) + 4 * g + (r & 3);
-                if (nn < W) out[(size_t)p * W + nn] = ((acc[r] + red[0][r][lane]) + red[1][r][lane]) + red[2][r][lane];
+                for (int r = 0; r < 16; ++r) red[wave - 1][r][lane] = acc[t][0][r];
             }
+            __syncthreads();
+            const int p = pb + 32 * t + c;
+            if (wave == 0 && p < p1) {
+#pragma unroll
+                for (int r = 0; r < 16; ++r) {
+                    const int nn = n0 + 8 * (r >> 2) + 4 * g + (r & 3);
+                    if (nn < W) out[(size_t)p * W + nn] = ((acc[t][0][r] + red[0][r][lane]) + red[1][r][lane]) + red[2][r][lane];
+                }
+            }
+            __syncthreads();
         }
-        __syncthreads();
     }
 }
 
