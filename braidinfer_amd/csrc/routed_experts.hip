@@ -530,26 +530,28 @@ extern "C" int br_experts_combine(const float* out, const int* place, const floa
 // ------------------------------------------- few tokens, every expert read once -----
 // bfloat16 on the matrix cores, for steps whose pairs were grouped by `sort` on the device (nothing comes back to
 // the host, so the step can be recorded): a workgroup owns 32 output rows of one expert's matrix and walks that
-// expert's pairs 64 at a time (as two tiles of 32, or one where no more are left), so an expert's weights are read once
-// per 64 of its pairs instead of once per pair.  Its four waves share k in runs of 64 (wave w takes the runs w, w + 4,
-// ...: the four loads a lane makes of a row's run fall into one line of 128 bytes, one after the other),
+// expert's pairs in tiles of 32, so an expert's weights are read once for a tile's pairs instead of once per pair; in
+// steps of more than 32 tokens two tiles at a time (where an expert has more than 32 pairs: few experts have, but those
+// would end last).  Its four waves share k in runs of 16 KS (wave w takes the runs w, w + 4, ...),
 // v_mfma_f32_32x32x16_bf16 with the weight rows as the first operand, both operands straight from memory; the waves'
 // sums meet in LDS in wave order.  Experts without pairs cost a workgroup a load and a compare.
+// One tile and runs of 16 keep the registers few and the waves many (32 experts of 1,792 by 4,096, 8 tokens: 242 us
+// `up` where two tiles and runs of 64 take 277); with two tiles runs of 32 are a little better than 16 or 64.
 
-// acc[tile][matrix] += the run-of-64 share of this wave: NM weight rows `w` (one a matrix) against the pairs' rows `a`
-// of one or two tiles.  Rows of the operands beyond the matrix's or the expert's last give results that nobody reads;
-// elements beyond K are zeros.
-template <int NM, int NT>
+// acc[tile][matrix] += the share of this wave (its runs of 16 KS along k): NM weight rows `w` (one a matrix) against the
+// pairs' rows `a` of NT tiles.  Rows of the operands beyond the matrix's or the expert's last give results that nobody
+// reads; elements beyond K are zeros.
+template <int KS, int NM, int NT>
 __device__ __forceinline__ void rx_walk(const bf16* const (&w)[NM], const bf16* const (&a)[NT], int K, int wave, int g,
                                         f32x16 (&acc)[2][NM]) {
     bf16x8 zero;
 #pragma unroll
     for (int i = 0; i < 8; ++i) zero[i] = (bf16)0.f;
-    for (int k0 = wave * 64; k0 < K; k0 += 256) {
-        bf16x8 wf[NM][4], af[NT][4];
-        const bool whole = k0 + 64 <= K;
+    for (int k0 = wave * 16 * KS; k0 < K; k0 += 64 * KS) {
+        bf16x8 wf[NM][KS], af[NT][KS];
+        const bool whole = k0 + 16 * KS <= K;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
+        for (int j = 0; j < KS; ++j) {
             const int k = k0 + 16 * j + 8 * g;
             const bool on = whole || k < K;
             const int kk = on ? k : 0;
@@ -562,7 +564,7 @@ __device__ __forceinline__ void rx_walk(const bf16* const (&w)[NM], const bf16* 
             }
         }
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
+        for (int j = 0; j < KS; ++j)
 #pragma unroll
             for (int t = 0; t < NT; ++t)
 #pragma unroll
@@ -573,6 +575,7 @@ __device__ __forceinline__ void rx_walk(const bf16* const (&w)[NM], const bf16* 
 
 // `up`: rows of h gathered through `order` (pair -> token = pair / top), gate and up rows of the same f in the same
 // lane, y[p, f] = silu(g) * u (or the clamped unit) in the experts' order.  grid (E, ceil(F / 32)).
+template <int TILES, int KS>
 __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __restrict__ h, const bf16* __restrict__ w_gu,
                                                                  const int* __restrict__ first, const int* __restrict__ order,
                                                                  bf16* __restrict__ y, int W, int F, int top, float limit, float alpha) {
@@ -585,8 +588,8 @@ __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __r
     const int f = f0 + c;
     const bf16* wg = w_gu + ((size_t)e * 2 * F + (f < F ? f : F - 1)) * W;
     const bf16* const w[2] = {wg, wg + (size_t)F * W};
-    for (int pb = p0; pb < p1; pb += 64) {
-        const bool two = pb + 32 < p1;
+    for (int pb = p0; pb < p1; pb += 32 * TILES) {
+        const bool two = TILES == 2 && pb + 32 < p1;
         f32x16 acc[2][2];
 #pragma unroll
         for (int t = 0; t < 2; ++t)
@@ -596,13 +599,13 @@ __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __r
         const bf16* a0 = h + (size_t)(order[pa] / top) * W;
         if (two) {
             const bf16* const a[2] = {a0, h + (size_t)(order[pz] / top) * W};
-            rx_walk<2, 2>(w, a, W, wave, g, acc);
+            rx_walk<KS, 2, 2>(w, a, W, wave, g, acc);
         } else {
             const bf16* const a[1] = {a0};
-            rx_walk<2, 1>(w, a, W, wave, g, acc);
+            rx_walk<KS, 2, 1>(w, a, W, wave, g, acc);
         }
 #pragma unroll
-        for (int t = 0; t < 2; ++t) {
+        for (int t = 0; t < TILES; ++t) {
             if (t == 1 && !two) break;
             if (wave > 0) {
 #pragma unroll
@@ -626,6 +629,7 @@ __global__ __launch_bounds__(256) void experts_up_grouped_kernel(const bf16* __r
 
 // `down`: out[p, n] = W_d[e] y[p, :] as float for the pairs in the experts' order (`combine` adds them to the rows).
 // grid (E, ceil(W / 32)).
+template <int TILES, int KS>
 __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* __restrict__ y, const bf16* __restrict__ w_down,
                                                                    const int* __restrict__ first, float* __restrict__ out,
                                                                    int W, int F) {
@@ -637,8 +641,8 @@ __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* _
     const int c = lane & 31, g = lane >> 5;
     const int n = n0 + c;
     const bf16* const w[1] = {w_down + ((size_t)e * W + (n < W ? n : W - 1)) * F};
-    for (int pb = p0; pb < p1; pb += 64) {
-        const bool two = pb + 32 < p1;
+    for (int pb = p0; pb < p1; pb += 32 * TILES) {
+        const bool two = TILES == 2 && pb + 32 < p1;
         f32x16 acc[2][1];
 #pragma unroll
         for (int t = 0; t < 2; ++t)
@@ -647,13 +651,13 @@ __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* _
         const bf16* a0 = y + (size_t)min(pb + c, p1 - 1) * F;
         if (two) {
             const bf16* const a[2] = {a0, y + (size_t)min(pb + 32 + c, p1 - 1) * F};
-            rx_walk<1, 2>(w, a, F, wave, g, acc);
+            rx_walk<KS, 1, 2>(w, a, F, wave, g, acc);
         } else {
             const bf16* const a[1] = {a0};
-            rx_walk<1, 1>(w, a, F, wave, g, acc);
+            rx_walk<KS, 1, 1>(w, a, F, wave, g, acc);
         }
 #pragma unroll
-        for (int t = 0; t < 2; ++t) {
+        for (int t = 0; t < TILES; ++t) {
             if (t == 1 && !two) break;
             if (wave > 0) {
 #pragma unroll
@@ -677,16 +681,20 @@ __global__ __launch_bounds__(256) void experts_down_grouped_kernel(const bf16* _
 extern "C" int br_experts_grouped_takes(int W, int F) { return W > 0 && F > 0 && W % 8 == 0 && F % 8 == 0; }
 
 extern "C" int br_experts_up_grouped(const void* h, const void* w_gu, const int* first, const int* order, void* y, int E,
-                                     int W, int F, int top, float limit, float alpha, hipStream_t s) {
+                                     int W, int F, int top, int n_tokens, float limit, float alpha, hipStream_t s) {
     if (!br_experts_grouped_takes(W, F) || E <= 0 || top <= 0 || (F + 31) / 32 > 65535) return BR_BAD_ARG;
-    experts_up_grouped_kernel<<<dim3(E, (F + 31) / 32), 256, 0, s>>>((const bf16*)h, (const bf16*)w_gu, first, order, (bf16*)y, W, F, top, limit, alpha);
+    const dim3 grid(E, (F + 31) / 32);
+    if (n_tokens <= 32) experts_up_grouped_kernel<1, 1><<<grid, 256, 0, s>>>((const bf16*)h, (const bf16*)w_gu, first, order, (bf16*)y, W, F, top, limit, alpha);
+    else experts_up_grouped_kernel<2, 2><<<grid, 256, 0, s>>>((const bf16*)h, (const bf16*)w_gu, first, order, (bf16*)y, W, F, top, limit, alpha);
     return br_check_launch();
 }
 
 extern "C" int br_experts_down_grouped(const void* y, const void* w_down, const int* first, float* out, int E, int W, int F,
-                                       hipStream_t s) {
+                                       int n_tokens, hipStream_t s) {
     if (!br_experts_grouped_takes(W, F) || E <= 0 || (W + 31) / 32 > 65535) return BR_BAD_ARG;
-    experts_down_grouped_kernel<<<dim3(E, (W + 31) / 32), 256, 0, s>>>((const bf16*)y, (const bf16*)w_down, first, out, W, F);
+    const dim3 grid(E, (W + 31) / 32);
+    if (n_tokens <= 32) experts_down_grouped_kernel<1, 1><<<grid, 256, 0, s>>>((const bf16*)y, (const bf16*)w_down, first, out, W, F);
+    else experts_down_grouped_kernel<2, 2><<<grid, 256, 0, s>>>((const bf16*)y, (const bf16*)w_down, first, out, W, F);
     return br_check_launch();
 }
 

@@ -1232,20 +1232,20 @@ def experts_up_grouped(h: torch.Tensor, w_gu: torch.Tensor, first: torch.Tensor,
     _req(experts_grouped_takes(h.dtype, W, F2 // 2) and w_gu.dtype == y.dtype == torch.bfloat16, "experts_up_grouped: bfloat16, widths in steps of 8")
     _req(w_gu.shape == (E, F2, W) and y.shape == (n, F2 // 2) and first.numel() in (E + 1, E + 2) and n == T * top
          and first.dtype == order.dtype == torch.int32, "experts_up_grouped: shapes")
-    f = _fn("routed_experts", "br_experts_up_grouped", [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_float, _P])
-    _check(f(_ptr(h), _ptr(w_gu), _ptr(first), _ptr(order), _ptr(y), E, W, F2 // 2, top, float(limit), float(alpha), _stream()),
+    f = _fn("routed_experts", "br_experts_up_grouped", [_P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P])
+    _check(f(_ptr(h), _ptr(w_gu), _ptr(first), _ptr(order), _ptr(y), E, W, F2 // 2, top, T, float(limit), float(alpha), _stream()),
            "experts_up_grouped")
 
 
-def experts_down_grouped(y: torch.Tensor, w_down: torch.Tensor, first: torch.Tensor, out: torch.Tensor) -> None:
-    """out[p] = W_down[e] y[p] (float) for the pairs in the experts' order."""
+def experts_down_grouped(y: torch.Tensor, w_down: torch.Tensor, first: torch.Tensor, out: torch.Tensor, n_tokens: int) -> None:
+    """out[p] = W_down[e] y[p] (float) for the pairs of `n_tokens` tokens in the experts' order (no expert has more pairs than that)."""
     _dev("experts_down_grouped", y, w_down, first, out)
     n, F = y.shape
     E, W, _ = w_down.shape
     _req(experts_grouped_takes(y.dtype, W, F) and w_down.dtype == torch.bfloat16 and out.dtype == torch.float32, "experts_down_grouped: types")
     _req(w_down.shape == (E, W, F) and out.shape == (n, W) and first.numel() in (E + 1, E + 2) and first.dtype == torch.int32, "experts_down_grouped: shapes")
-    f = _fn("routed_experts", "br_experts_down_grouped", [_P, _P, _P, _P, c_int, c_int, c_int, _P])
-    _check(f(_ptr(y), _ptr(w_down), _ptr(first), _ptr(out), E, W, F, _stream()), "experts_down_grouped")
+    f = _fn("routed_experts", "br_experts_down_grouped", [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P])
+    _check(f(_ptr(y), _ptr(w_down), _ptr(first), _ptr(out), E, W, F, int(n_tokens), _stream()), "experts_down_grouped")
 
 
 def experts_gemm(a: torch.Tensor, w: torch.Tensor, first: torch.Tensor, out: torch.Tensor) -> None:

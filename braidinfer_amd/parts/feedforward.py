@@ -285,7 +285,7 @@ class RoutedExperts(FeedForward):
             y = step.ws.get("moe_y", (n, self.I), dt)
             K.experts_up_grouped(h, self.w_gu, first, order, y, self.top, self.limit, self.alpha)
             out = step.ws.get("moe_out", (n, self.H), torch.float32)
-            K.experts_down_grouped(y, self.w_down, first, out)
+            K.experts_down_grouped(y, self.w_down, first, out, T)
             K.experts_combine(out, place, share, x, store=store, **ident)
             return
         rows = step.ws.get("moe_rows", (n, self.H), dt)

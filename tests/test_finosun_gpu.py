@@ -465,7 +465,7 @@ def test_many_pairs_of_one_expert(n_pairs):
     y = torch.zeros((T, F), dtype=torch.bfloat16, device="cuda")
     K.experts_up_grouped(dev_16(h), dev_16(gu), first, order, y, 1, 0.7, 1.702)
     out = torch.zeros((T, W), device="cuda")
-    K.experts_down_grouped(y, dev_16(down), first, out)
+    K.experts_down_grouped(y, dev_16(down), first, out, T)
     x = torch.full((T, W), 3.0, device="cuda")
     share = dev_f(np.linspace(0.5, 1.5, T)[:, None])
     K.experts_combine(out, place, share, x, chosen=chosen, h=dev_16(h), experts=E, store=True)

@@ -366,7 +366,7 @@ def test_routing_and_experts():
             K.experts_up_grouped(hd, w_gu, first, order, y2, top)
             assert np.abs(y2[place.long()].float().cpu().numpy().reshape(T, top, F) - y.float().cpu().numpy()).max() < 0.02 * float(y.float().abs().max())
             out = torch.zeros((n, W), dtype=torch.float32, device="cuda")
-            K.experts_down_grouped(y2, stack("down"), first, out)
+            K.experts_down_grouped(y2, stack("down"), first, out, T)
             x2 = torch.tensor(x0).cuda()
             K.experts_combine(out, place, share, x2)
             assert np.abs(x2.cpu().numpy() - x0 - want).max() < tol * max(1.0, np.abs(want).max())
