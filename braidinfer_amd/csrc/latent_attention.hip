@@ -98,6 +98,9 @@ extern "C" int br_latent_prepare(const float* q, size_t q_stride, const float* d
 // token in four neighbouring registers), both operands straight from memory 16 bytes a lane; four waves a
 // workgroup side by side along n.  grid (ceil(T / 32), ceil(N / 128), H).  K in steps of 8, rows and heads of a
 // at multiples of 16 bytes.
+// VEC: a lane's four neighbouring n go out (and its gates come in) as one vector: N, the output's strides and the gate's
+// in steps of 4, aligned.
+template <bool VEC>
 __global__ __launch_bounds__(256) void head_linear_bf16_kernel(const bf16* __restrict__ a, size_t lda, size_t a_hs,
                                                                const bf16* __restrict__ w, bf16* __restrict__ out, size_t ldo,
                                                                size_t o_hs, const float* __restrict__ gate, size_t gate_stride,
@@ -123,6 +126,20 @@ __global__ __launch_bounds__(256) void head_linear_bf16_kernel(const bf16* __res
     }
     if (t >= T) return;
     bf16* orow = out + (size_t)t * ldo + (size_t)h * o_hs;
+    if (VEC) {
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+            const int n = n0 + 8 * q + 4 * g;
+            if (n >= N) continue;
+            f32x4 z = {0.f, 0.f, 0.f, 0.f};
+            if (gate) z = *(const f32x4*)(gate + (size_t)t * gate_stride + (size_t)h * N + n);
+            bf16x4 o;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = (bf16)(gate ? acc[4 * q + e] / (1.0f + expf(-z[e])) : acc[4 * q + e]);
+            *(bf16x4*)(orow + n) = o;
+        }
+        return;
+    }
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
         const int n = n0 + 8 * (r >> 2) + 4 * g + (r & 3);
@@ -158,7 +175,9 @@ extern "C" int br_head_linear(const void* a, size_t lda, size_t a_hs, const void
     if ((gate && gate_stride < (size_t)H * N) || H <= 0 || N <= 0 || K <= 0 || H > 65535 || (N + 127) / 128 > 65535) return BR_BAD_ARG;
     if (is_bf16 && K % 8 == 0 && lda % 8 == 0 && a_hs % 8 == 0 && ((uintptr_t)a % 16) == 0 && ((uintptr_t)w % 16) == 0) {
         dim3 grid((T + 31) / 32, (N + 127) / 128, H);
-        head_linear_bf16_kernel<<<grid, 256, 0, s>>>((const bf16*)a, lda, a_hs, (const bf16*)w, (bf16*)out, ldo, o_hs, gate, gate_stride, T, N, K);
+        const bool vec = N % 4 == 0 && ldo % 4 == 0 && o_hs % 4 == 0 && gate_stride % 4 == 0 && ((uintptr_t)out % 8) == 0 && ((uintptr_t)gate % 16) == 0;
+        if (vec) head_linear_bf16_kernel<true><<<grid, 256, 0, s>>>((const bf16*)a, lda, a_hs, (const bf16*)w, (bf16*)out, ldo, o_hs, gate, gate_stride, T, N, K);
+        else head_linear_bf16_kernel<false><<<grid, 256, 0, s>>>((const bf16*)a, lda, a_hs, (const bf16*)w, (bf16*)out, ldo, o_hs, gate, gate_stride, T, N, K);
         return br_check_launch();
     }
     const size_t n = (size_t)T * H * N;
