@@ -452,7 +452,7 @@ def test_many_pairs_of_one_expert(n_pairs):
     pairs of identities behind them."""
     from braidinfer_amd import kernels as K
     rng = np.random.default_rng(n_pairs)
-    E, W, F = 4, 136, 72                                 # k runs that end inside a run of 64
+    E, W, F = 4, 136, 72                                 # both inner lengths end inside a run along k
     T = n_pairs + 3
     h = bf(rng.standard_normal((T, W)))
     gu, down = bf(rng.standard_normal((E, 2 * F, W)) / math.sqrt(W)), bf(rng.standard_normal((E, W, F)) / math.sqrt(F))
