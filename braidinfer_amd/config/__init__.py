@@ -8,11 +8,13 @@ from .sidirax import SidiraxConfig, build_spec as build_sidirax_spec, ARCHITECTU
 from .zivovik import ZivovikConfig, build_spec as build_zivovik_spec, ARCHITECTURE as ZIVOVIK
 from .ladadra import LadadraConfig, build_spec as build_ladadra_spec, ARCHITECTURE as LADADRA
 from .finosun import FinosunConfig, build_spec as build_finosun_spec, ARCHITECTURE as FINOSUN
+from .tuzisun import TuzisunConfig, build_spec as build_tuzisun_spec, ARCHITECTURE as TUZISUN
 from . import finosun as _finosun
 from . import kesitar as _kesitar
 from . import ladadra as _ladadra
 from . import zivovik as _zivovik
 from . import sidirax as _sidirax
+from . import tuzisun as _tuzisun
 
 register_architecture(MISTRAL, MistralConfig, build_mistral_spec, model_type="mistral", replace=True)
 register_architecture(KESITAR, KesitarConfig, build_kesitar_spec, model_type="kesitar", replace=True)
@@ -20,9 +22,11 @@ register_architecture(SIDIRAX, SidiraxConfig, build_sidirax_spec, model_type="si
 register_architecture(ZIVOVIK, ZivovikConfig, build_zivovik_spec, model_type="zivovik", replace=True)
 register_architecture(LADADRA, LadadraConfig, build_ladadra_spec, model_type="ladadra", replace=True)
 register_architecture(FINOSUN, FinosunConfig, build_finosun_spec, model_type="finosun", replace=True)
+register_architecture(TUZISUN, TuzisunConfig, build_tuzisun_spec, model_type="tuzisun", replace=True)
 PRESET_FAMILIES = {MISTRAL: (PRESETS, preset), KESITAR: (_kesitar.PRESETS, _kesitar.preset),
                    SIDIRAX: (_sidirax.PRESETS, _sidirax.preset), ZIVOVIK: (_zivovik.PRESETS, _zivovik.preset),
-                   LADADRA: (_ladadra.PRESETS, _ladadra.preset), FINOSUN: (_finosun.PRESETS, _finosun.preset)}
+                   LADADRA: (_ladadra.PRESETS, _ladadra.preset), FINOSUN: (_finosun.PRESETS, _finosun.preset),
+                   TUZISUN: (_tuzisun.PRESETS, _tuzisun.preset)}
 
 
 def any_preset(name: str, **overrides):
@@ -38,5 +42,5 @@ __all__ = [
     "Architecture", "register_architecture", "unregister_architecture", "registered_architectures",
     "architecture_of", "architecture_of_config", "read_config_json", "config_from_dict",
     "config_from_folder", "spec_of", "generation_stop_tokens", "MistralConfig", "PRESETS", "preset",
-    "KesitarConfig", "SidiraxConfig", "ZivovikConfig", "LadadraConfig", "FinosunConfig", "any_preset", "PRESET_FAMILIES",
+    "KesitarConfig", "SidiraxConfig", "ZivovikConfig", "LadadraConfig", "FinosunConfig", "TuzisunConfig", "any_preset", "PRESET_FAMILIES",
 ]

@@ -54,6 +54,9 @@ class LayerSpec:
     # the block arrangement the layer names is what runs them (`mixer_ctx.others[role]`).  Their tensor-name
     # pieces are `names["mixer.<role>"]`, their cache units `ScheduleEntry.more_caches[role]`.
     more_mixers: Dict[str, PartSpec] = field(default_factory=dict)
+    # what couples the halves to a residual of several streams (`ModelSpec.streams`), by the half's role ("mixer",
+    # "feed_forward"); tensor-name pieces `names["connection.<role>"]`, run by the arrangement the layer names
+    connections: Dict[str, PartSpec] = field(default_factory=dict)
 
     def name_of(self, what: str) -> str:
         if what not in self.names:
@@ -127,6 +130,9 @@ class ModelSpec:
     # of each one's tensors (absent: "join.<name>.")
     input_joins: Dict[str, PartSpec] = field(default_factory=dict)
     input_join_prefixes: Dict[str, str] = field(default_factory=dict)
+    # residual rows kept as this many streams side by side, all equal to the embedding output at first and summed in front
+    # of the final norm; None: one row a token.  The layers' arrangements must be made for streams.
+    streams: Optional[int] = None
     # tensors a checkpoint may carry that no part reads (a norm in front of a feed-forward the layer does not have)
     optional_tensors: List[str] = field(default_factory=list)
 

@@ -41,6 +41,7 @@ MODULES: Dict[str, List[str]] = {
     "delta_rule": ["delta_rule.hip"],
     "latent_attention": ["latent_attention.hip"],
     "routed_experts": ["routed_experts.hip"],
+    "streams": ["streams.hip"],
 }
 HEADERS = ["common.h", "no_alloc.h"]
 

@@ -78,3 +78,25 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
     for (int i = 0; i < nw; ++i) t += scratch[i];
     return t;
 }
+
+// VEC (4 or 1) neighbouring elements as floats; 4: one aligned load or store.
+template <typename T> struct ew_vec4;
+template <> struct ew_vec4<float> { typedef f32x4 type; };
+template <> struct ew_vec4<bf16> { typedef bf16x4 type; };
+template <typename T, int VEC>
+__device__ __forceinline__ void ew_load(const T* p, float* v) {
+    if (VEC == 4) {
+        const typename ew_vec4<T>::type q = *(const typename ew_vec4<T>::type*)p;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = to_f32<T>(q[e]);
+    } else v[0] = to_f32<T>(p[0]);
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void ew_store(T* p, const float* v) {
+    if (VEC == 4) {
+        typename ew_vec4<T>::type q;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) q[e] = from_f32<T>(v[e]);
+        *(typename ew_vec4<T>::type*)p = q;
+    } else p[0] = from_f32<T>(v[0]);
+}

@@ -519,26 +519,6 @@ extern "C" int br_silu_mul(const void* gu, void* a, int is_bf16, int T, int I, h
 // their roundings) and the biases b [2 I] (null: none); a has the products' type.  `row_gate` (null: none): a number a
 // row, `gate_stride` elements apart; the row is multiplied by its sigmoid.  VEC 4: four elements a thread (I in steps
 // of 4, aligned buffers).
-template <typename T> struct ew_vec4;
-template <> struct ew_vec4<float> { typedef f32x4 type; };
-template <> struct ew_vec4<bf16> { typedef bf16x4 type; };
-template <typename T, int VEC>
-__device__ __forceinline__ void ew_load(const T* p, float* v) {
-    if (VEC == 4) {
-        const typename ew_vec4<T>::type q = *(const typename ew_vec4<T>::type*)p;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = to_f32<T>(q[e]);
-    } else v[0] = to_f32<T>(p[0]);
-}
-template <typename T, int VEC>
-__device__ __forceinline__ void ew_store(T* p, const float* v) {
-    if (VEC == 4) {
-        typename ew_vec4<T>::type q;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) q[e] = from_f32<T>(v[e]);
-        *(typename ew_vec4<T>::type*)p = q;
-    } else p[0] = from_f32<T>(v[0]);
-}
 template <typename TG, typename T, int VEC>
 __global__ void clamped_glu_kernel(const TG* __restrict__ gu, const float* __restrict__ b, const float* __restrict__ row_gate,
                                    size_t gate_stride, T* __restrict__ a, int I, size_t n, float limit, float alpha) {
@@ -661,30 +641,30 @@ extern "C" int br_convert(const void* a, void* b, int to_bf16, size_t n, hipStre
     return br_check_launch();
 }
 
-// out[t, i] = x[t, i] for float rows x [T, H], in out's type; out's rows lie `ldo` elements apart (a column range of
-// wider rows).  VEC: four elements a thread (H and ldo in steps of 4, aligned).
+// out[t, i] = x[t, i] for float rows x [T, H], in out's type; x's rows lie `ldx` and out's `ldo` elements apart (column
+// ranges of wider rows).  VEC: four elements a thread (H, ldx and ldo in steps of 4, aligned).
 template <typename T, int VEC>
-__global__ void rows_into_kernel(const float* __restrict__ x, T* __restrict__ out, int H, size_t ldo, size_t n) {
+__global__ void rows_into_kernel(const float* __restrict__ x, size_t ldx, T* __restrict__ out, int H, size_t ldo, size_t n) {
     const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= n) return;
     const size_t t = i / H, c = i - t * H;
     float v[VEC];
-    ew_load<float, VEC>(x + i, v);
+    ew_load<float, VEC>(x + t * ldx + c, v);
     ew_store<T, VEC>(out + t * ldo + c, v);
 }
 
-extern "C" int br_rows_into(const float* x, void* out, int is_bf16, int T, int H, size_t ldo, hipStream_t s) {
+extern "C" int br_rows_into(const float* x, size_t ldx, void* out, int is_bf16, int T, int H, size_t ldo, hipStream_t s) {
     if (T <= 0) return BR_OK;
-    if (H <= 0 || ldo < (size_t)H) return BR_BAD_ARG;
+    if (H <= 0 || ldo < (size_t)H || ldx < (size_t)H) return BR_BAD_ARG;
     const size_t n = (size_t)T * H;
-    const bool vec = H % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0;
+    const bool vec = H % 4 == 0 && ldo % 4 == 0 && ldx % 4 == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0;
     const unsigned blocks = (unsigned)(((vec ? n / 4 : n) + 255) / 256);
     if (is_bf16) {
-        if (vec) rows_into_kernel<bf16, 4><<<blocks, 256, 0, s>>>(x, (bf16*)out, H, ldo, n);
-        else rows_into_kernel<bf16, 1><<<blocks, 256, 0, s>>>(x, (bf16*)out, H, ldo, n);
+        if (vec) rows_into_kernel<bf16, 4><<<blocks, 256, 0, s>>>(x, ldx, (bf16*)out, H, ldo, n);
+        else rows_into_kernel<bf16, 1><<<blocks, 256, 0, s>>>(x, ldx, (bf16*)out, H, ldo, n);
     } else {
-        if (vec) rows_into_kernel<float, 4><<<blocks, 256, 0, s>>>(x, (float*)out, H, ldo, n);
-        else rows_into_kernel<float, 1><<<blocks, 256, 0, s>>>(x, (float*)out, H, ldo, n);
+        if (vec) rows_into_kernel<float, 4><<<blocks, 256, 0, s>>>(x, ldx, (float*)out, H, ldo, n);
+        else rows_into_kernel<float, 1><<<blocks, 256, 0, s>>>(x, ldx, (float*)out, H, ldo, n);
     }
     return br_check_launch();
 }

@@ -630,74 +630,122 @@ extern "C" int br_shift_mix(const void* h, int is_bf16, const float* mu, void* o
 // ------------------------------------------------ head norm, weight and gate --------
 // y[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) * w[h, :] * silu(gate[t, h, :]): every head's output
 // divided by its root mean square, a weight per head and channel, and a gate from the float sums of its
-// projection (rows `gate_stride` floats apart; `gate_sigmoid`: sigmoid of the sums instead of silu).  16 lanes a
-// (token, head) row as in `glr_head_norm_kernel`.
-template <typename T>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
-                                                             const float* __restrict__ gate, size_t gate_stride,
-                                                             T* __restrict__ y, size_t n_rows, int H, int e, float eps,
-                                                             int gate_sigmoid) {
+// projection (rows `gate_stride` floats apart; `gate_sigmoid`: sigmoid of the sums instead of silu).  `gate_first`: the
+// gate multiplies o ahead of the norm.  With `n` (float [T, H], the read-out of a memory's normaliser, beside `m` [T, H],
+// what the memory is kept relative to) o[t, h, :] is first multiplied by q_mul / (max(|n q_mul|, exp(-m)) + 1e-6).
+// 16 lanes a (token, head) row as in `glr_head_norm_kernel`; V4: four channels a lane at a time (e, the gate's stride
+// and all pointers in steps of 16 bytes).
+struct HeadNormGate {
+    const float *o, *w, *gate, *n, *m;
+    size_t gate_stride;
+    int H, e, gate_sigmoid, gate_first;
+    float eps, q_mul;
+};
+
+__device__ __forceinline__ float hng_gate(float z, int sigmoid) { return (sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
+__device__ __forceinline__ float hng_scale(const HeadNormGate& p, size_t r) {
+    return p.n ? p.q_mul / (fmaxf(fabsf(p.n[r] * p.q_mul), expf(-p.m[r])) + 1e-6f) : 1.0f;
+}
+
+template <typename T, bool V4>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const HeadNormGate p, T* __restrict__ y, size_t n_rows) {
+    constexpr int V = V4 ? 4 : 1;
+    typedef float vec_t __attribute__((ext_vector_type(V)));
+    typedef T out_t __attribute__((ext_vector_type(V)));
     const size_t r = (size_t)blockIdx.x * 16 + (threadIdx.x >> 4);
-    const int l = threadIdx.x & 15;
+    const int l = threadIdx.x & 15, e = p.e, nv = e / V;
     const bool on = r < n_rows;
-    const float* orow = o + (on ? r : 0) * e;
+    const float* orow = p.o + (on ? r : 0) * e;
+    const size_t t = (on ? r : 0) / p.H;
+    const int hh = (int)((on ? r : 0) - t * p.H);
+    const float* grow = p.gate ? p.gate + t * p.gate_stride + (size_t)hh * e : nullptr;
+    const float* wrow = p.w ? p.w + (size_t)hh * e : nullptr;
+    const float scale = on ? hng_scale(p, r) : 1.0f;
+    const bool first = p.gate_first && grow;
     float ss = 0.f;
-    for (int i = l; i < e; i += 16) { const float v = on ? orow[i] : 0.f; ss += v * v; }
-    const float inv = 1.0f / sqrtf(glr_row16_sum(ss) / (float)e + eps);
+    for (int i = l; i < nv; i += 16) {
+        vec_t v = ((const vec_t*)orow)[i], z;
+        if (first) z = ((const vec_t*)grow)[i];
+#pragma unroll
+        for (int x = 0; x < V; ++x) {
+            float f = ((const float*)&v)[x] * scale;
+            if (first) f *= hng_gate(((const float*)&z)[x], p.gate_sigmoid);
+            ss = fmaf(f, f, ss);
+        }
+    }
+    const float inv = 1.0f / sqrtf(glr_row16_sum(on ? ss : 0.f) / (float)e + p.eps);
     if (!on) return;
-    const size_t t = r / H;
-    const int hh = (int)(r - t * H);
-    const float* grow = gate ? gate + t * gate_stride + (size_t)hh * e : nullptr;
-    const float* wrow = w ? w + (size_t)hh * e : nullptr;
     T* yrow = y + r * e;
-    for (int i = l; i < e; i += 16) {
-        float v = orow[i] * inv;
-        if (wrow) v *= wrow[i];
-        if (grow) { const float z = grow[i]; v *= (gate_sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
-        yrow[i] = from_f32<T>(v);
+    for (int i = l; i < nv; i += 16) {
+        const vec_t v = ((const vec_t*)orow)[i];
+        vec_t wv, z;
+        if (wrow) wv = ((const vec_t*)wrow)[i];
+        if (grow) z = ((const vec_t*)grow)[i];
+        out_t out;
+#pragma unroll
+        for (int x = 0; x < V; ++x) {
+            float f = ((const float*)&v)[x] * scale * inv;
+            if (wrow) f *= ((const float*)&wv)[x];
+            if (grow) f *= hng_gate(((const float*)&z)[x], p.gate_sigmoid);
+            ((T*)&out)[x] = from_f32<T>(f);
+        }
+        ((out_t*)yrow)[i] = out;
     }
 }
 
 // The same for rows of many channels (all heads normed together, say): a workgroup a (token, head) row.
 template <typename T>
-__global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(const float* __restrict__ o, const float* __restrict__ w,
-                                                                  const float* __restrict__ gate, size_t gate_stride,
-                                                                  T* __restrict__ y, int H, int e, float eps, int gate_sigmoid) {
+__global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(const HeadNormGate p, T* __restrict__ y) {
     __shared__ float scratch[16];
     const size_t r = blockIdx.x;
-    const float* orow = o + r * e;
+    const int e = p.e;
+    const float* orow = p.o + r * e;
+    const size_t t = r / p.H;
+    const int hh = (int)(r - t * p.H);
+    const float* grow = p.gate ? p.gate + t * p.gate_stride + (size_t)hh * e : nullptr;
+    const float* wrow = p.w ? p.w + (size_t)hh * e : nullptr;
+    const float scale = hng_scale(p, r);
+    const bool first = p.gate_first && grow;
     float ss = 0.f;
-    for (int i = threadIdx.x; i < e; i += 256) { const float v = orow[i]; ss = fmaf(v, v, ss); }
-    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)e + eps);
-    const size_t t = r / H;
-    const int hh = (int)(r - t * H);
-    const float* grow = gate ? gate + t * gate_stride + (size_t)hh * e : nullptr;
-    const float* wrow = w ? w + (size_t)hh * e : nullptr;
+    for (int i = threadIdx.x; i < e; i += 256) {
+        float v = orow[i] * scale;
+        if (first) v *= hng_gate(grow[i], p.gate_sigmoid);
+        ss = fmaf(v, v, ss);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)e + p.eps);
     T* yrow = y + r * e;
     for (int i = threadIdx.x; i < e; i += 256) {
-        float v = orow[i] * inv;
+        float v = orow[i] * scale * inv;
         if (wrow) v *= wrow[i];
-        if (grow) { const float z = grow[i]; v *= (gate_sigmoid ? 1.0f : z) / (1.0f + expf(-z)); }
+        if (grow) v *= hng_gate(grow[i], p.gate_sigmoid);
         yrow[i] = from_f32<T>(v);
     }
 }
 
 #define HNG_WIDE_FROM 512      // channels of a row from which a workgroup takes it
 
-extern "C" int br_head_norm_gate(const float* o, const float* w, const float* gate, size_t gate_stride, void* y, int y_is_bf16,
-                                 int T, int H, int e, float eps, int gate_sigmoid, hipStream_t s) {
+extern "C" int br_head_norm_gate(const float* o, const float* w, const float* gate, size_t gate_stride, const float* n, const float* m,
+                                 float q_mul, void* y, int y_is_bf16, int T, int H, int e, float eps, int gate_sigmoid, int gate_first,
+                                 hipStream_t s) {
     if (T <= 0) return BR_OK;
-    if (H <= 0 || e <= 0 || (gate && gate_stride < (size_t)H * e)) return BR_BAD_ARG;
+    if (H <= 0 || e <= 0 || (gate && gate_stride < (size_t)H * e) || (!n != !m)) return BR_BAD_ARG;
     const size_t n_rows = (size_t)T * H;
+    const HeadNormGate p = {o, w, gate, n, m, gate_stride, H, e, gate_sigmoid, gate_first, eps, q_mul};
     if (e >= HNG_WIDE_FROM) {
         if (n_rows > 0x7fffffffULL) return BR_BAD_ARG;
-        if (y_is_bf16) head_norm_gate_wide_kernel<bf16><<<(unsigned)n_rows, 256, 0, s>>>(o, w, gate, gate_stride, (bf16*)y, H, e, eps, gate_sigmoid);
-        else head_norm_gate_wide_kernel<float><<<(unsigned)n_rows, 256, 0, s>>>(o, w, gate, gate_stride, (float*)y, H, e, eps, gate_sigmoid);
+        if (y_is_bf16) head_norm_gate_wide_kernel<bf16><<<(unsigned)n_rows, 256, 0, s>>>(p, (bf16*)y);
+        else head_norm_gate_wide_kernel<float><<<(unsigned)n_rows, 256, 0, s>>>(p, (float*)y);
         return br_check_launch();
     }
     const unsigned blocks = (unsigned)((n_rows + 15) / 16);
-    if (y_is_bf16) head_norm_gate_kernel<bf16><<<blocks, 256, 0, s>>>(o, w, gate, gate_stride, (bf16*)y, n_rows, H, e, eps, gate_sigmoid);
-    else head_norm_gate_kernel<float><<<blocks, 256, 0, s>>>(o, w, gate, gate_stride, (float*)y, n_rows, H, e, eps, gate_sigmoid);
+    const bool v4 = e % 4 == 0 && gate_stride % 4 == 0 && (((uintptr_t)o | (uintptr_t)w | (uintptr_t)gate | (uintptr_t)y) % 16) == 0;
+    if (y_is_bf16) {
+        if (v4) head_norm_gate_kernel<bf16, true><<<blocks, 256, 0, s>>>(p, (bf16*)y, n_rows);
+        else head_norm_gate_kernel<bf16, false><<<blocks, 256, 0, s>>>(p, (bf16*)y, n_rows);
+    } else {
+        if (v4) head_norm_gate_kernel<float, true><<<blocks, 256, 0, s>>>(p, (float*)y, n_rows);
+        else head_norm_gate_kernel<float, false><<<blocks, 256, 0, s>>>(p, (float*)y, n_rows);
+    }
     return br_check_launch();
 }
 

@@ -107,7 +107,7 @@ __device__ __forceinline__ void route_scores(const float* __restrict__ zrow, int
 
 // Routing by scores with a choice correction and groups of experts.  s = sigmoid(z), or (SOFTMAX) the softmax of z over
 // all outputs; the choice is made on c = s + correction, the shares on s.  A token's logits lie `ld` elements apart.  With `groups` > 1 the experts form that many runs of E / groups neighbours; a
-// run's score is the sum of its two largest c (of its one, where a run is one expert), only experts of the `keep`
+// run's score is the sum of its two largest c (of its one, where a run is one expert, or always with `run_max`), only experts of the `keep`
 // best runs can be chosen (the others count as minus infinity), ties to the lower number everywhere.  The shares are
 // the chosen experts' s over their sum (+ 1e-20), or as they are without `renorm`, times `out_scale`.  grid (T), one wave
 // a token.
@@ -118,7 +118,7 @@ __device__ __forceinline__ void route_scores(const float* __restrict__ zrow, int
 template <int NPL, bool SOFTMAX>
 __global__ __launch_bounds__(64) void route_corrected_kernel(const float* __restrict__ scores, int ld, const float* __restrict__ correction,
                                                              int* __restrict__ chosen, float* __restrict__ share, int E, int top,
-                                                             int groups, int keep, int renorm, float out_scale) {
+                                                             int groups, int keep, int run_max, int renorm, float out_scale) {
     extern __shared__ float rs_lds[];
     float* cs = rs_lds;                     // [E] the choice scores
     float* gsL = cs + E;                    // [groups] the runs' scores, then whether a run is kept
@@ -152,7 +152,7 @@ __global__ __launch_bounds__(64) void route_corrected_kernel(const float* __rest
                     const float v = cs[g * per + i];
                     if (v > b1) { b2 = b1; b1 = v; } else if (v > b2) b2 = v;
                 }
-                gs[j] = per > 1 ? b1 + b2 : b1;
+                gs[j] = per > 1 && !run_max ? b1 + b2 : b1;
                 gsL[g] = gs[j];
             }
         }
@@ -212,7 +212,7 @@ __global__ __launch_bounds__(64) void route_corrected_kernel(const float* __rest
 template <bool SOFTMAX>
 __global__ __launch_bounds__(64) void route_corrected_rounds_kernel(const float* __restrict__ scores, int ld, const float* __restrict__ correction,
                                                                     int* __restrict__ chosen, float* __restrict__ share, int E, int top,
-                                                                    int groups, int keep, int renorm, float out_scale) {
+                                                                    int groups, int keep, int run_max, int renorm, float out_scale) {
     extern __shared__ float cs[];           // the choice scores
     const int t = blockIdx.x, lane = threadIdx.x;
     float sg[RX_MAX_PER_LANE], z[RX_MAX_PER_LANE];
@@ -241,7 +241,7 @@ __global__ __launch_bounds__(64) void route_corrected_rounds_kernel(const float*
                     const float v = cs[g * per + i];
                     if (v > b1) { b2 = b1; b1 = v; } else if (v > b2) b2 = v;
                 }
-                gs[j] = per > 1 ? b1 + b2 : b1;
+                gs[j] = per > 1 && !run_max ? b1 + b2 : b1;
             }
         }
         __syncthreads();
@@ -300,17 +300,17 @@ __global__ __launch_bounds__(64) void route_corrected_rounds_kernel(const float*
     if (lane < top) share[(size_t)t * top + lane] = (renorm ? mine / (total + 1e-20f) : mine) * out_scale;
 }
 
-// `softmax`: s is the softmax over all E outputs, else the sigmoid; `renorm`: the shares are divided by their sum.
+// `run_max`: a run's score is its largest c alone; `softmax`: s is the softmax over all E outputs, else the sigmoid; `renorm`: the shares are divided by their sum.
 extern "C" int br_route_corrected(const float* scores, int ld, const float* correction, int* chosen, float* share, int T, int E, int top,
-                                  int groups, int keep, int softmax, int renorm, float out_scale, hipStream_t s) {
+                                  int groups, int keep, int run_max, int softmax, int renorm, float out_scale, hipStream_t s) {
     if (T <= 0) return BR_OK;
     if (E <= 0 || E > 64 * RX_MAX_PER_LANE || top <= 0 || top > E || top > 64 || groups <= 0 || E % groups || ld < E ||
         (groups > 1 && (keep <= 0 || keep > groups)))
         return BR_BAD_ARG;
     const size_t lds = (size_t)(E + groups + 128) * sizeof(float), lds_rounds = (size_t)E * sizeof(float);
 #define RX_ROUTE(SM) do { \
-        if (E <= 64) route_corrected_kernel<1, SM><<<T, 64, lds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, renorm, out_scale); \
-        else route_corrected_rounds_kernel<SM><<<T, 64, lds_rounds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, renorm, out_scale); \
+        if (E <= 64) route_corrected_kernel<1, SM><<<T, 64, lds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, run_max, renorm, out_scale); \
+        else route_corrected_rounds_kernel<SM><<<T, 64, lds_rounds, s>>>(scores, ld, correction, chosen, share, E, top, groups, keep, run_max, renorm, out_scale); \
     } while (0)
     if (softmax) RX_ROUTE(true); else RX_ROUTE(false);
 #undef RX_ROUTE

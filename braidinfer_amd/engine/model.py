@@ -32,10 +32,13 @@ class Layer:
         self.more_mixers: Dict[str, object] = {role: build_part("mixer", ms) for role, ms in spec.more_mixers.items()}
         self.feed_forward = build_part("feed_forward", spec.feed_forward) if spec.feed_forward else None
         self.norms: Dict[str, object] = {role: build_part("norm", ns) for role, ns in spec.norms.items()}
+        self.connections: Dict[str, object] = {role: build_part("connection", cs) for role, cs in spec.connections.items()}
         arrangement = block_arrangement(spec.block)
         # an arrangement is an object with `run` (and optionally `first_norm`), or a plain function
         self.run = getattr(arrangement, "run", arrangement)
         self._first_norm = getattr(arrangement, "first_norm", None)
+        self._opening = getattr(arrangement, "opening", None)
+        self.takes_streams = bool(getattr(arrangement, "takes_streams", False))
         self.rt: Optional[Runtime] = None
 
     # the two norms of the common arrangement, by their roles
@@ -52,6 +55,10 @@ class Layer:
         arrangement says."""
         return self._first_norm(self) if self._first_norm is not None else None
 
+    def opening(self):
+        """(connection, norm) through which the layer's first half reads a residual of several streams, or None."""
+        return self._opening(self) if self._opening is not None else None
+
     def named_parts(self):
         """(part, tensor-name prefix) in the order of the spec's `names`, which is the order
         of the layer's tensors in the model's name table."""
@@ -65,15 +72,18 @@ class Layer:
                 part = self.norms.get(what[5:])
             elif what.startswith("mixer."):
                 part = self.more_mixers.get(what[6:])
+            elif what.startswith("connection."):
+                part = self.connections.get(what[11:])
             else:
                 raise ConfigError(f"layer {s.prefix!r}: names has {what!r}; known: mixer, mixer.<role>, feed_forward, "
-                                  "norm.<role>")
+                                  "norm.<role>, connection.<role>")
             if part is not None:
                 yield part, s.name_of(what)
         named = set(s.names)
         missing = [w for w, p in [("mixer", self.mixer), ("feed_forward", self.feed_forward)]
                    + [("norm." + r, n) for r, n in self.norms.items()]
-                   + [("mixer." + r, m) for r, m in self.more_mixers.items()] if p is not None and w not in named]
+                   + [("mixer." + r, m) for r, m in self.more_mixers.items()]
+                   + [("connection." + r, c) for r, c in self.connections.items()] if p is not None and w not in named]
         if missing:
             raise ConfigError(f"layer {s.prefix!r}: no tensor-name piece for {missing}")
 
@@ -94,6 +104,12 @@ class DecoderModel:
             if e.input_join is not None and e.input_join not in self.input_joins:
                 raise ConfigError(f"schedule entry of layer {e.layer} names the input join {e.input_join!r}, the model has "
                                   f"{sorted(self.input_joins)}")
+        if spec.streams is not None and (int(spec.streams) < 1 or any(e.adds_embedding or e.input_join for e in self.schedule)):
+            raise ConfigError(f"a residual of {spec.streams} streams: at least one, and no entry of the run order may join the embedding in")
+        for e in self.schedule:
+            if self.layers[e.layer].takes_streams != (spec.streams is not None):
+                raise ConfigError(f"layer {e.layer}: the arrangement {self.layers[e.layer].spec.block!r} does not go with a residual of "
+                                  f"{'one row a token' if spec.streams is None else f'{spec.streams} streams'}")
         written = set()
         for e in self.schedule:
             if e.cache is not None and self.layers[e.layer].mixer is not None:
@@ -256,6 +272,11 @@ class DecoderModel:
         for join in self.input_joins.values():
             join.begin(x, step)
         step.prepared_norm = None
+        S = self.spec.streams
+        if S is not None and S > 1:
+            streams = ws.get("residual_streams", (T, S * H), torch.float32)
+            K.streams_spread(x, streams, S)
+            x = streams
         for i, e in enumerate(self.schedule):
             layer = self.layers[e.layer]
             step.schedule_index = i
@@ -268,6 +289,7 @@ class DecoderModel:
             # the norm that reads the residual rows after this layer: the next scheduled layer's first
             # (the final norm reads chosen rows only and is left alone)
             step.norm_after_layer = None
+            step.next_layer = self.layers[self.schedule[i + 1].layer] if i + 1 < len(self.schedule) else None
             if i + 1 < len(self.schedule) and self.schedule[i + 1].input_join is None:
                 step.norm_after_layer = self.layers[self.schedule[i + 1].layer].first_norm()
             ctx = (self._mixer_context(cache, e, i, None) if layer.mixer is not None
@@ -285,7 +307,16 @@ class DecoderModel:
         if n_want == 0:
             return logits
         hn = ws.get("final_h", (n_want, H), rt.dtype)
-        self.final_norm.forward(x, hn, rows=want_rows)
+        if S is not None and S > 1:
+            point = self.final_norm.point_args()
+            if point is not None:          # the streams' sum and the norm of it in one pass
+                K.streams_open(x, hn, S, norm=point, rows=want_rows)
+            else:
+                total = ws.get("streams_sum", (n_want, H), torch.float32)
+                K.streams_open(x, total, S, rows=want_rows)
+                self.final_norm.forward(total, hn)
+        else:
+            self.final_norm.forward(x, hn, rows=want_rows)
         if probe is not None:
             probe("final_norm", hn)
         self.lm_head.forward(hn, logits, ws)

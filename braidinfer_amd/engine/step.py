@@ -58,6 +58,7 @@ class StepBatch:
     # between the parts of a step: the norm that reads the residual rows after the running layer, and
     # what the last product into the rows prepared for a norm, as (norm, rows, preparation)
     norm_after_layer: Any = None
+    next_layer: Any = None           # the layer that runs after the running one, or None
     prepared_norm: Any = None
     extras: Dict[str, Any] = field(default_factory=dict)     # per-step scratch of parts (keyed by them)
     # what the position encodings read: [T], the same tensor as `positions` unless the caller gave

@@ -144,13 +144,72 @@ def layernorm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, eps: float, r
 
 
 def rows_into(x: torch.Tensor, out: torch.Tensor) -> None:
-    """out = x in out's dtype: x float [T, H] dense, out [T, H] with dense rows that may lie further apart (a range of
-    columns of wider rows)."""
-    _dev("rows_into", x)
+    """out[t, :] = x[t, :] in out's dtype; x is float [T, H]; the rows of both may be strided (column ranges of wider buffers)."""
+    _req(x.is_cuda and out.is_cuda and x.dtype == torch.float32 and x.dim() == 2 and out.shape == x.shape and x.stride(1) == 1
+         and out.stride(1) == 1, "rows_into: x float32 [T, H], out [T, H] with dense rows, on the GPU")
     T, H = x.shape
-    _req(x.dtype == torch.float32 and out.is_cuda and out.shape == (T, H) and out.stride(1) == 1, "rows_into: x float32 [T, H], out [T, H] with dense rows")
-    f = _fn("elementwise", "br_rows_into", [_P, _P, c_int, c_int, c_int, c_size_t, _P])
-    _check(f(_ptr(x), _ptr(out), _is_bf16(out, "rows_into"), T, H, out.stride(0) if T > 1 else H, _stream()), "rows_into")
+    f = _fn("elementwise", "br_rows_into", [_P, c_size_t, _P, c_int, c_int, c_int, c_size_t, _P])
+    _check(f(_ptr(x), x.stride(0) if T > 1 else H, _ptr(out), _is_bf16(out, "rows_into"), T, H, out.stride(0) if T > 1 else H,
+             _stream()), "rows_into")
+
+
+# ------------------------------------------------------------- residual streams -----
+def _point_norm(name: str, norm, W: int):
+    """(alpha, weight, bias) of a norm tanh(alpha u) w + b as pointers, or nulls."""
+    if norm is None:
+        return c_void_p(0), c_void_p(0), c_void_p(0)
+    alpha, w, b = norm
+    _dev(name, alpha, w, b)
+    _req(alpha.dtype == w.dtype == b.dtype == torch.float32 and alpha.numel() == 1 and w.numel() == W and b.numel() == W,
+         f"{name}: a norm's alpha [1], weight and bias [W], float32")
+    return _ptr(alpha), _ptr(w), _ptr(b)
+
+
+def streams_spread(x: torch.Tensor, X: torch.Tensor, S: int) -> None:
+    """X[t] = x[t] side by side S times: every stream of a token starts as its row.  x float [T, W], X float [T, S * W]."""
+    _dev("streams_spread", x, X)
+    T, W = x.shape
+    _req(x.dtype == X.dtype == torch.float32 and X.shape == (T, S * W) and 1 <= S <= 16, "streams_spread: float32 [T, W] and [T, S W], 1..16 streams")
+    f = _fn("streams", "br_streams_spread", [_P, _P, c_int, c_int, c_int, _P])
+    _check(f(_ptr(x), _ptr(X), T, S, W, _stream()), "streams_spread")
+
+
+def streams_open(X: torch.Tensor, h: torch.Tensor, S: int, weights: Optional[torch.Tensor] = None, norm=None,
+                 rows: Optional[torch.Tensor] = None) -> None:
+    """h[r] = norm(sum_s weights[s] X[rows[r]][s]): `weights` float [S] (None: ones), `norm` (alpha, w, b) for
+    tanh(alpha u) w + b (None: none), `rows` int32 [R] (None: every row in order)."""
+    _dev("streams_open", X, h, weights, rows)
+    R, W = h.shape
+    _req(X.dtype == torch.float32 and X.dim() == 2 and X.shape[1] == S * W and 1 <= S <= 16, "streams_open: X float32 [T, S W], 1..16 streams")
+    _req(weights is None or (weights.dtype == torch.float32 and weights.numel() >= S), "streams_open: weights float32 [S]")
+    _req(X.shape[0] == R if rows is None else (rows.dtype == torch.int32 and rows.numel() == R), "streams_open: rows int32 [R], or h of X's rows")
+    f = _fn("streams", "br_streams_open", [_P] * 7 + [c_int] * 4 + [_P])
+    _check(f(_ptr(X), _ptr(rows), _ptr(weights), *_point_norm("streams_open", norm, W), _ptr(h), _is_bf16(h, "streams_open"), R, S, W,
+             _stream()), "streams_open")
+
+
+def streams_join(X: torch.Tensor, coef: torch.Tensor, branches, S: int, h: Optional[torch.Tensor] = None,
+                 next_weights: Optional[torch.Tensor] = None, norm=None) -> None:
+    """X_t <- sum_s mix[s, t] X_s + out[t] y in place, `coef` float in [S] | out [S] | mix [S, S] (mix is indexed [from, to]) and
+    y the sum over one or two `branches` (rows float [T, W], bias float [W] or None, scale) of scale (rows + bias).  With `h`
+    [T, W]: h = norm(sum_s next_weights[s] X_s) of the new streams, in the same pass (`next_weights`, `norm` as in
+    `streams_open`)."""
+    T = X.shape[0]
+    _req(1 <= len(branches) <= 2, "streams_join: one or two branches")
+    W = branches[0][0].shape[1]
+    _dev("streams_join", X, coef, h, next_weights, *[t for r, b, _ in branches for t in (r, b)])
+    _req(X.dtype == torch.float32 and X.shape == (T, S * W) and 1 <= S <= 16, "streams_join: X float32 [T, S W], 1..16 streams")
+    _req(coef.dtype == torch.float32 and coef.numel() == 2 * S + S * S, "streams_join: coef float32 [S + S + S S]")
+    for r, b, _ in branches:
+        _req(r.dtype == torch.float32 and r.shape == (T, W) and (b is None or (b.dtype == torch.float32 and b.numel() == W)),
+             "streams_join: a branch's rows float32 [T, W] and bias float32 [W]")
+    _req(h is None or h.shape == (T, W), "streams_join: h [T, W]")
+    _req(next_weights is None or (next_weights.dtype == torch.float32 and next_weights.numel() >= S), "streams_join: next_weights float32 [S]")
+    (y1, b1, s1), (y2, b2, s2) = branches[0], (branches[1] if len(branches) == 2 else (None, None, 0.0))
+    f = _fn("streams", "br_streams_join", [_P, _P, _P, _P, c_float, _P, _P, c_float, _P, _P, _P, _P, _P] + [c_int] * 4 + [_P])
+    _check(f(_ptr(X), _ptr(coef), _ptr(y1), _ptr(b1), float(s1), _ptr(y2), _ptr(b2), float(s2), _ptr(next_weights),
+             *_point_norm("streams_join", norm, W), _ptr(h), 0 if h is None else _is_bf16(h, "streams_join"), T, S, W, _stream()),
+           "streams_join")
 
 
 def scale_(x: torch.Tensor, scale: float) -> None:
@@ -901,9 +960,11 @@ def shift_mix(h: torch.Tensor, mu: torch.Tensor, out: torch.Tensor, kept: torch.
 
 
 def head_norm_gate(o: torch.Tensor, w: Optional[torch.Tensor], gate: Optional[torch.Tensor], out: torch.Tensor, H: int, e: int,
-                   eps: float, gate_sigmoid: bool = False) -> None:
+                   eps: float, gate_sigmoid: bool = False, gate_first: bool = False, normaliser=None) -> None:
     """out[t, h, :] = o[t, h, :] / rms * w[h, :] * silu(gate[t, h, :]) (`gate_sigmoid`: sigmoid instead of silu): o float
-    [T, H*e], w float [H*e] or None, gate a float view [T, H*e] whose rows may be strided (the sums of its projection) or None."""
+    [T, H*e], w float [H*e] or None, gate a float view [T, H*e] whose rows may be strided (the sums of its projection) or None.
+    `gate_first`: o is multiplied by the gate ahead of the norm.  `normaliser` (n, m, q_mul), n and m float [T, H]:
+    o[t, h, :] is first multiplied by q_mul / (max(|n q_mul|, exp(-m)) + 1e-6)."""
     _dev("head_norm_gate", o, w, out)
     T = o.shape[0]
     _req(o.dtype == torch.float32 and o.shape == (T, H * e) and out.shape == (T, H * e), "head_norm_gate: o float32 [T, H*e]")
@@ -912,70 +973,155 @@ def head_norm_gate(o: torch.Tensor, w: Optional[torch.Tensor], gate: Optional[to
     if gate is not None:
         _req(gate.is_cuda and gate.dtype == torch.float32 and gate.shape == (T, H * e) and gate.stride(1) == 1, "head_norm_gate: gate float32 [T, H*e]")
         gs = gate.stride(0) if T > 1 else H * e
-    f = _fn("gated_recurrence", "br_head_norm_gate", [_P, _P, _P, c_size_t, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P])
-    _check(f(_ptr(o), _ptr(w), _ptr(gate), gs, _ptr(out), _is_bf16(out, "head_norm_gate"), T, H, e, float(eps),
-             int(bool(gate_sigmoid)), _stream()), "head_norm_gate")
+    n = m = None
+    q_mul = 1.0
+    if normaliser is not None:
+        n, m, q_mul = normaliser
+        _dev("head_norm_gate", n, m)
+        _req(n.dtype == m.dtype == torch.float32 and n.shape == m.shape == (T, H), "head_norm_gate: the normaliser's read-out and maxima float32 [T, H]")
+    f = _fn("gated_recurrence", "br_head_norm_gate", [_P, _P, _P, c_size_t, _P, _P, c_float, _P, c_int, c_int, c_int, c_int, c_float, c_int, c_int, _P])
+    _check(f(_ptr(o), _ptr(w), _ptr(gate), gs, _ptr(n), _ptr(m), float(q_mul), _ptr(out), _is_bf16(out, "head_norm_gate"), T, H, e, float(eps),
+             int(bool(gate_sigmoid)), int(bool(gate_first)), _stream()), "head_norm_gate")
 
 
 # ------------------------------------------------- recurrences with one decay a head -----
+def _kept_inputs(name: str, kept: Optional[torch.Tensor], n: int, C: int) -> int:
+    """The slot stride of a convolution's kept inputs, float view [slots, (n - 1) * C]; 0 where one tap keeps nothing."""
+    if n <= 1:
+        return 0
+    _req(kept is not None and kept.is_cuda and kept.dtype == torch.float32 and kept.dim() == 2 and kept.shape[1] == (n - 1) * C
+         and kept.stride(1) == 1, f"{name}: kept float32 [slots, (n - 1) * C]")
+    return kept.stride(0)
+
+
 def dr_conv_prepare(rows: torch.Tensor, taps: torch.Tensor, kept: Optional[torch.Tensor], a_log: torch.Tensor,
                     dt_bias: torch.Tensor, seq_of_token: torch.Tensor, cu_seqlens: torch.Tensor, slots: torch.Tensor,
                     q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gb: torch.Tensor, B: int, G: int, H: int, d: int,
-                    e: int, taps_t: Optional[torch.Tensor] = None) -> None:
-    """rows float [T, >= C + 2 H] with C = 2 G d + H e: the sums q | k | v | b | a of a gated delta rule's projections.
-    The first C columns pass a causal convolution over time per channel (taps float [C, n], the last column the current
-    token's; `kept` a float view [slots, (n - 1) * C] of every sequence's last inputs, read and then brought up to
-    date) and silu; q and k become unit vectors per head (q times d^-1/2); gb [T, 2 H] takes
+                    e: int, taps_t: Optional[torch.Tensor] = None, decay: Optional[torch.Tensor] = None,
+                    gc: Optional[torch.Tensor] = None, single_tokens: bool = False) -> None:
+    """rows float [T, >= C + 2 H] with C = 2 G d + H e (a view whose rows may be strided): the sums q | k | v | b | a of a
+    gated delta rule's projections.  The first C columns pass a causal convolution over time per channel (taps float [C, n],
+    the last column the current token's; `kept` a float view [slots, (n - 1) * C] of every sequence's last inputs, read and
+    then brought up to date) and silu; q and k become unit vectors per head (q times d^-1/2); gb [T, 2 H] takes
     g = exp(-exp(a_log) softplus(a + dt_bias)) and beta = sigmoid(b).  `taps_t` float [n, C], the same taps with the channels
-    side by side, lets widths that are multiples of 4 go four channels a lane."""
-    _dev("dr_conv_prepare", rows, taps, a_log, dt_bias, seq_of_token, cu_seqlens, slots, q, k, v, gb, taps_t)
+    side by side, lets widths that are multiples of 4 go four channels a lane.  With `decay` (a float view [T, H d]) there
+    is one decay a head and key channel: rows have no a, dt_bias is [H d], gc [T, H d] takes
+    exp(-exp(a_log) softplus(decay + dt_bias)) and gb's first half is left alone.  `single_tokens`: every sequence brings
+    one token (one launch less)."""
+    _dev("dr_conv_prepare", taps, a_log, dt_bias, seq_of_token, cu_seqlens, slots, q, k, v, gb, taps_t, gc)
     T = rows.shape[0]
     C = 2 * G * d + H * e
     n = taps.shape[1] if taps.dim() == 2 else 0
-    _req(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[1] >= C + 2 * H, "dr_conv_prepare: rows float32 [T, >= C + 2 H]")
+    behind = H if decay is not None else 2 * H
+    _req(rows.is_cuda and rows.dtype == torch.float32 and rows.dim() == 2 and rows.stride(1) == 1 and rows.shape[1] >= C + behind,
+         "dr_conv_prepare: rows float32 [T, >= C + 2 H]")
     _req(taps.dtype == torch.float32 and taps.shape == (C, n) and 1 <= n <= 16, "dr_conv_prepare: taps float32 [C, 1..16]")
-    _req(a_log.dtype == dt_bias.dtype == torch.float32 and a_log.numel() == H and dt_bias.numel() == H, "dr_conv_prepare: A_log and dt_bias float32 [H]")
+    _req(a_log.dtype == dt_bias.dtype == torch.float32 and a_log.numel() == H and dt_bias.numel() == (H if decay is None else H * d),
+         "dr_conv_prepare: A_log float32 [H], dt_bias float32 [H] (or [H d])")
     _req(q.dtype == k.dtype == v.dtype == gb.dtype == torch.float32 and q.shape == k.shape == (T, G * d) and v.shape == (T, H * e)
          and gb.shape == (T, 2 * H), "dr_conv_prepare: q, k [T, G d], v [T, H e], gb [T, 2 H] float32")
     _req(seq_of_token.numel() >= T and cu_seqlens.numel() >= B + 1 and slots.numel() >= B, "dr_conv_prepare: arrays shorter than the batch")
-    ks = 0
-    if n > 1:
-        _req(kept is not None and kept.is_cuda and kept.dtype == torch.float32 and kept.dim() == 2 and kept.shape[1] == (n - 1) * C
-             and kept.stride(1) == 1, "dr_conv_prepare: kept float32 [slots, (n - 1) * C]")
-        ks = kept.stride(0)
+    _req((decay is None) == (gc is None) and (decay is None or (decay.is_cuda and decay.dtype == gc.dtype == torch.float32 and decay.stride(1) == 1
+         and decay.shape == gc.shape == (T, H * d))), "dr_conv_prepare: decay and gc float32 [T, H d] come together")
+    ks = _kept_inputs("dr_conv_prepare", kept, n, C)
     _req(taps_t is None or (taps_t.dtype == torch.float32 and taps_t.shape == (n, C) and taps_t.is_contiguous()), "dr_conv_prepare: taps_t float32 [n, C]")
-    f = _fn("delta_rule", "br_dr_conv_prepare", [_P, c_int, _P, _P, c_int, _P, c_size_t, _P, _P, _P, _P, _P, _P, _P, _P, _P] + [c_int] * 6 + [_P])
-    _check(f(_ptr(rows), int(rows.shape[1]), _ptr(taps), _ptr(taps_t), n, _ptr(kept) if n > 1 else c_void_p(0), ks, _ptr(a_log), _ptr(dt_bias),
-             _ptr(seq_of_token), _ptr(cu_seqlens), _ptr(slots), _ptr(q), _ptr(k), _ptr(v), _ptr(gb), T, B, G, H, d, e, _stream()),
-           "dr_conv_prepare")
+    zs = 0 if decay is None else (decay.stride(0) if T > 1 else H * d)
+    f = _fn("delta_rule", "br_dr_conv_prepare", [_P, c_int, _P, _P, c_int, _P, c_size_t] + [_P] * 10 + [c_size_t, _P] + [c_int] * 7 + [_P])
+    _check(f(_ptr(rows), int(rows.stride(0) if T > 1 else rows.shape[1]), _ptr(taps), _ptr(taps_t), n, _ptr(kept) if n > 1 else c_void_p(0), ks,
+             _ptr(a_log), _ptr(dt_bias), _ptr(seq_of_token), _ptr(cu_seqlens), _ptr(slots), _ptr(q), _ptr(k), _ptr(v), _ptr(gb), _ptr(decay), zs,
+             _ptr(gc), T, B, G, H, d, e, int(bool(single_tokens)), _stream()), "dr_conv_prepare")
+
+
+def ssm_prepare(x: torch.Tensor, taps_t: torch.Tensor, bias: Optional[torch.Tensor], kept: Optional[torch.Tensor], dt: torch.Tensor,
+                a_log: torch.Tensor, dt_bias: torch.Tensor, seq_of_token: torch.Tensor, cu_seqlens: torch.Tensor, slots: torch.Tensor,
+                out: torch.Tensor, gb: torch.Tensor, B: int, single_tokens: bool = False) -> None:
+    """out [T, C] = silu(causal convolution over time of x per channel + bias): x a float view [T, C], taps_t float [n, C] (the
+    current token's last), `kept` as in `dr_conv_prepare`.  dt a float view [T, H] of the same row stride: gb [T, 2 H] takes
+    exp(-exp(a_log) s) and s = softplus(dt + dt_bias).  `single_tokens`: every sequence brings one token."""
+    _dev("ssm_prepare", taps_t, bias, a_log, dt_bias, seq_of_token, cu_seqlens, slots, out, gb)
+    T, C = x.shape
+    H, n = dt.shape[1], taps_t.shape[0]
+    for t in (x, dt):
+        _req(t.is_cuda and t.dtype == torch.float32 and t.dim() == 2 and t.shape[0] == T and t.stride(1) == 1, "ssm_prepare: x [T, C] and dt [T, H] float32 with dense rows")
+    _req(T <= 1 or x.stride(0) == dt.stride(0), "ssm_prepare: rows of x and dt equally far apart")
+    _req(taps_t.dtype == torch.float32 and taps_t.shape == (n, C) and 1 <= n <= 16, "ssm_prepare: taps_t float32 [1..16, C]")
+    _req(bias is None or (bias.dtype == torch.float32 and bias.numel() == C), "ssm_prepare: bias float32 [C]")
+    _req(a_log.dtype == dt_bias.dtype == torch.float32 and a_log.numel() == dt_bias.numel() == H, "ssm_prepare: A_log and dt_bias float32 [H]")
+    _req(out.dtype == gb.dtype == torch.float32 and out.shape == (T, C) and gb.shape == (T, 2 * H), "ssm_prepare: out [T, C], gb [T, 2 H] float32")
+    _req(seq_of_token.numel() >= T and cu_seqlens.numel() >= B + 1 and slots.numel() >= B, "ssm_prepare: arrays shorter than the batch")
+    ks = _kept_inputs("ssm_prepare", kept, n, C)
+    f = _fn("delta_rule", "br_ssm_prepare", [_P, c_size_t, _P, _P, c_int, _P, c_size_t] + [_P] * 8 + [c_int] * 5 + [_P])
+    _check(f(_ptr(x), x.stride(0) if T > 1 else max(C, H), _ptr(taps_t), _ptr(bias), n, _ptr(kept) if n > 1 else c_void_p(0), ks, _ptr(dt),
+             _ptr(a_log), _ptr(dt_bias), _ptr(seq_of_token), _ptr(cu_seqlens), _ptr(slots), _ptr(out), _ptr(gb), T, B, C, H,
+             int(bool(single_tokens)), _stream()), "ssm_prepare")
+
+
+def exp_gates(zi: torch.Tensor, zf: torch.Tensor, bi: torch.Tensor, bf: torch.Tensor, cap: float, kept: torch.Tensor,
+              cu_seqlens: torch.Tensor, slots: torch.Tensor, gb: torch.Tensor, m: torch.Tensor, B: int) -> None:
+    """Exponential input and sigmoid forget gates over a running maximum: i = cap tanh((zi + bi) / cap),
+    f = log sigmoid(cap tanh((zf + bf) / cap)), m_t = max(f + m_(t-1), i) from the slot's kept m (float view [slots, H], left
+    behind); gb [T, 2 H] takes exp(f + m_(t-1) - m_t) and exp(i - m_t), m [T, H] the maxima.  zi, zf float views [T, H]."""
+    _dev("exp_gates", bi, bf, cu_seqlens, slots, gb, m)
+    T, H = zi.shape
+    for t in (zi, zf):
+        _req(t.is_cuda and t.dtype == torch.float32 and t.shape == (T, H) and t.stride(1) == 1, "exp_gates: sums float32 [T, H]")
+    _req(T <= 1 or zi.stride(0) == zf.stride(0), "exp_gates: rows of both sums equally far apart")
+    _req(bi.dtype == bf.dtype == torch.float32 and bi.numel() == bf.numel() == H and cap > 0, "exp_gates: biases float32 [H], a positive bound")
+    _req(kept.is_cuda and kept.dtype == torch.float32 and kept.dim() == 2 and kept.shape[1] == H and kept.stride(1) == 1, "exp_gates: kept float32 [slots, H]")
+    _req(gb.dtype == m.dtype == torch.float32 and gb.shape == (T, 2 * H) and m.shape == (T, H), "exp_gates: gb [T, 2 H], m [T, H] float32")
+    _req(cu_seqlens.numel() >= B + 1 and slots.numel() >= B, "exp_gates: arrays shorter than the batch")
+    f = _fn("delta_rule", "br_exp_gates", [_P, _P, c_size_t, _P, _P, c_float, _P, c_size_t, _P, _P, _P, _P, c_int, c_int, _P])
+    _check(f(_ptr(zi), _ptr(zf), zi.stride(0) if T > 1 else H, _ptr(bi), _ptr(bf), float(cap), _ptr(kept), kept.stride(0), _ptr(cu_seqlens),
+             _ptr(slots), _ptr(gb), _ptr(m), B, H, _stream()), "exp_gates")
+
+
+_DR_FIXED, _DR_DELTA, _DR_WEIGHTED, _DR_CHANNELS = range(4)
+
+
+def _dr_scan_check(name, q, k, v, gb, decay, gc, weighted, skip, n_out, out, state, cu, slots, B, H, G, d, e, silu) -> int:
+    """The checks `dr_scan` and `dr_scan_pieces` share; returns the kernels' mode."""
+    _dev(name, gb, decay, gc, skip, n_out, out, cu, slots)
+    T = out.shape[0]
+    for what, t, w in (("q", q, G * d), ("k", k, G * d), ("v", v, H * e)):
+        _req(t.is_cuda and t.dtype == torch.float32 and t.shape == (T, w) and t.stride(1) == 1, f"{name}: {what} float32 [T, {w}]")
+    _req(T <= 1 or q.stride(0) == k.stride(0), f"{name}: q and k rows equally far apart")
+    _req((gb is None) != (decay is None), f"{name}: either numbers per token or one decay a head")
+    _req(gb is None or (gb.dtype == torch.float32 and gb.shape == (T, 2 * H)), f"{name}: gb float32 [T, 2 H]")
+    _req(decay is None or (decay.dtype == torch.float32 and decay.numel() == H), f"{name}: decay float32 [H]")
+    _req(gc is None or (gb is not None and not weighted and gc.dtype == torch.float32 and gc.shape == (T, H * d)),
+         f"{name}: decays of key channels float32 [T, H d] go with the delta rule")
+    _req(not weighted or gb is not None, f"{name}: a weighted sum takes gb")
+    _req((skip is None and n_out is None) or weighted, f"{name}: skip and n_out go with the weighted sum")
+    _req(skip is None or (skip.dtype == torch.float32 and skip.numel() == H), f"{name}: skip float32 [H]")
+    _req(n_out is None or (n_out.dtype == torch.float32 and n_out.shape == (T, H)), f"{name}: n_out float32 [T, H]")
+    _req(not silu or decay is not None, f"{name}: silu goes with one decay a head")
+    _req(out.dtype == torch.float32 and out.shape == (T, H * e), f"{name}: out float32 [T, H e]")
+    _req(state.is_cuda and state.dtype == torch.float32 and tuple(state.shape[1:]) == tuple(glr_state_shape(H, d, e + (n_out is not None)))
+         and state[0].is_contiguous(), f"{name}: state float32 [slots, H, ceil(e/4), rows per lane, 64] (e + 1 columns with n_out), every slot's dense")
+    _req(slots.numel() >= B, f"{name}: arrays shorter than the batch")
+    _req(H % G == 0 and d <= 512, f"{name}: {H} heads over {G} key heads of {d} channels (a multiple; at most 512 channels)")
+    return _DR_FIXED if gb is None else (_DR_WEIGHTED if weighted else (_DR_CHANNELS if gc is not None else _DR_DELTA))
 
 
 def dr_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gb: Optional[torch.Tensor], decay: Optional[torch.Tensor],
             out: torch.Tensor, state: torch.Tensor, cu_seqlens: torch.Tensor, slots: torch.Tensor, B: int, H: int, G: int,
-            d: int, e: int, silu: bool = False) -> None:
+            d: int, e: int, silu: bool = False, gc: Optional[torch.Tensor] = None, weighted: bool = False,
+            skip: Optional[torch.Tensor] = None, n_out: Optional[torch.Tensor] = None) -> None:
     """A walk over every sequence's new tokens with a state S [d, e] a head, float, in `state` [slots, *glr_state_shape]
     (a view whose slots may be strided).  q, k float views [T, G d], v [T, H e] (rows may be strided; head h reads
     q/k head h // (H / G)).  With `gb` [T, 2 H] (g | beta) the gated delta rule
-    S <- g S; u = beta (v - S^T k); S <- S + k u^T; else with `decay` [H] S <- decay_h S + k v^T.  o = S^T q after
-    the write, into out float [T, H e].  `silu`: q, k, v pass silu on their way in."""
-    _dev("dr_scan", gb, decay, out, cu_seqlens, slots)
+    S <- g S; u = beta (v - S^T k); S <- S + k u^T (`gc` [T, H d]: one decay a key channel instead of g, diag(gc) S); with
+    `weighted` S <- g S + beta k v^T; else with `decay` [H] S <- decay_h S + k v^T.  o = S^T q after the write, into out
+    float [T, H e].  `silu` (with `decay`): q, k, v pass silu on their way in.  With `weighted`: `skip` [H] adds skip_h v to
+    o, and `n_out` [T, H] takes the read-out of one column more, whose value is 1 (the state is then [d, e + 1] a head)."""
+    mode = _dr_scan_check("dr_scan", q, k, v, gb, decay, gc, weighted, skip, n_out, out, state, cu_seqlens, slots, B, H, G, d, e, silu)
+    _req(cu_seqlens.numel() >= B + 1, "dr_scan: arrays shorter than the batch")
     T = out.shape[0]
-    for name, t, w in (("q", q, G * d), ("k", k, G * d), ("v", v, H * e)):
-        _req(t.is_cuda and t.dtype == torch.float32 and t.shape == (T, w) and t.stride(1) == 1, f"dr_scan: {name} float32 [T, {w}]")
-    _req(T <= 1 or q.stride(0) == k.stride(0), "dr_scan: q and k rows equally far apart")
-    _req((gb is None) != (decay is None), "dr_scan: either g and beta per token or one decay a head")
-    _req(gb is None or (gb.dtype == torch.float32 and gb.shape == (T, 2 * H)), "dr_scan: gb float32 [T, 2 H]")
-    _req(decay is None or (decay.dtype == torch.float32 and decay.numel() == H), "dr_scan: decay float32 [H]")
-    _req(out.dtype == torch.float32 and out.shape == (T, H * e), "dr_scan: out float32 [T, H e]")
-    _req(state.is_cuda and state.dtype == torch.float32 and tuple(state.shape[1:]) == tuple(glr_state_shape(H, d, e))
-         and state[0].is_contiguous(), "dr_scan: state float32 [slots, H, ceil(e/4), rows per lane, 64], every slot's dense")
-    _req(cu_seqlens.numel() >= B + 1 and slots.numel() >= B, "dr_scan: arrays shorter than the batch")
-    _req(H % G == 0 and d <= 512, f"dr_scan: {H} heads over {G} key heads of {d} channels (a multiple; at most 512 channels)")
     qs = q.stride(0) if T > 1 else G * d
     vs = v.stride(0) if T > 1 else H * e
-    f = _fn("delta_rule", "br_dr_scan", [_P, _P, c_size_t, _P, c_size_t, _P, c_size_t, _P, _P, _P, c_size_t, _P, _P] + [c_int] * 7 + [_P])
-    _check(f(_ptr(q), _ptr(k), qs, _ptr(v), vs, _ptr(gb), 2 * H, _ptr(decay), _ptr(out), _ptr(state), state.stride(0),
-             _ptr(cu_seqlens), _ptr(slots), B, H, G, d, e, int(gb is not None), int(bool(silu)), _stream()), "dr_scan")
+    f = _fn("delta_rule", "br_dr_scan", [_P, _P, c_size_t, _P, c_size_t, _P, c_size_t] + [_P] * 6 + [c_size_t, _P, _P] + [c_int] * 8 + [_P])
+    _check(f(_ptr(q), _ptr(k), qs, _ptr(v), vs, _ptr(gb), 2 * H, _ptr(decay), _ptr(gc), _ptr(skip), _ptr(out), _ptr(n_out), _ptr(state),
+             state.stride(0), _ptr(cu_seqlens), _ptr(slots), B, H, G, d, e, mode, int(n_out is not None), int(bool(silu)), _stream()), "dr_scan")
 
 
 def dr_rotate_rows(q: torch.Tensor, k: torch.Tensor, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], rotary_dim: int,
@@ -1005,32 +1151,32 @@ def silu_rows(x: torch.Tensor) -> None:
     _check(f(_ptr(x), x.stride(0) if T > 1 else n, T, n, _stream()), "silu_rows")
 
 
-def dr_scan_pieces(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, out: torch.Tensor, state: torch.Tensor,
+def dr_scan_pieces(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: Optional[torch.Tensor], out: torch.Tensor, state: torch.Tensor,
                    slots: torch.Tensor, piece_cu: torch.Tensor, piece_slots: torch.Tensor, piece_state: torch.Tensor, B: int,
-                   pieces: int, H: int, d: int, e: int, silu: bool = False) -> None:
-    """`dr_scan` with one decay a head over a step of long prompts with every sequence cut into `pieces` pieces that are
-    walked side by side (twice: from a zero state, then from their true first states).  `piece_cu` int32 [B*pieces + 1]
-    cuts the packed tokens, `piece_slots` int32 [B*pieces] numbers the pieces (-1: a padding sequence's); `piece_state`
-    float [B*pieces, *glr_state_shape] is scratch."""
-    _dev("dr_scan_pieces", decay, out, slots, piece_cu, piece_slots, piece_state)
+                   pieces: int, H: int, d: int, e: int, silu: bool = False, G: Optional[int] = None, gb: Optional[torch.Tensor] = None,
+                   skip: Optional[torch.Tensor] = None, n_out: Optional[torch.Tensor] = None, piece_decay: Optional[torch.Tensor] = None) -> None:
+    """`dr_scan` with one decay a head, or the weighted sum (`gb`, with `skip`, `n_out` as there), over a step of long prompts
+    with every sequence cut into `pieces` pieces that are walked side by side (twice: from a zero state, then from their true
+    first states).  `piece_cu` int32 [B*pieces + 1] cuts the packed tokens, `piece_slots` int32 [B*pieces] numbers the
+    pieces (-1: a padding sequence's); `piece_state` float [B*pieces, *glr_state_shape] and, with `gb`, `piece_decay` float
+    [B*pieces, H] are scratch."""
+    G = H if G is None else G
+    mode = _dr_scan_check("dr_scan_pieces", q, k, v, gb, decay, None, gb is not None, skip, n_out, out, state, piece_cu, slots, B, H, G, d, e, silu)
+    _dev("dr_scan_pieces", piece_slots, piece_state, piece_decay)
     T = out.shape[0]
-    shape = tuple(glr_state_shape(H, d, e))
-    for name, t, w in (("q", q, H * d), ("k", k, H * d), ("v", v, H * e)):
-        _req(t.is_cuda and t.dtype == torch.float32 and t.shape == (T, w) and t.stride(1) == 1, f"dr_scan_pieces: {name} float32 [T, {w}]")
-    _req(T <= 1 or q.stride(0) == k.stride(0), "dr_scan_pieces: q and k rows equally far apart")
-    _req(decay.dtype == torch.float32 and decay.numel() == H, "dr_scan_pieces: decay float32 [H]")
-    _req(out.dtype == torch.float32 and out.shape == (T, H * e), "dr_scan_pieces: out float32 [T, H e]")
-    _req(state.is_cuda and state.dtype == torch.float32 and tuple(state.shape[1:]) == shape and state[0].is_contiguous(),
-         "dr_scan_pieces: state float32 [slots, *glr_state_shape], every slot's dense")
+    shape = tuple(glr_state_shape(H, d, e + (n_out is not None)))
     _req(piece_state.dtype == torch.float32 and piece_state.shape == (B * pieces,) + shape and piece_state.is_contiguous(),
          "dr_scan_pieces: scratch of the wrong size")
-    _req(piece_cu.dtype == piece_slots.dtype == torch.int32 and piece_cu.numel() == B * pieces + 1 and piece_slots.numel() == B * pieces
-         and slots.numel() >= B, "dr_scan_pieces: piece arrays int32 [B*pieces + 1] and [B*pieces]")
-    qs = q.stride(0) if T > 1 else H * d
+    _req(gb is None or (piece_decay is not None and piece_decay.dtype == torch.float32 and piece_decay.numel() >= B * pieces * H),
+         "dr_scan_pieces: the weighted sum takes piece_decay float32 [B*pieces, H]")
+    _req(piece_cu.dtype == piece_slots.dtype == torch.int32 and piece_cu.numel() == B * pieces + 1 and piece_slots.numel() == B * pieces,
+         "dr_scan_pieces: piece arrays int32 [B*pieces + 1] and [B*pieces]")
+    qs = q.stride(0) if T > 1 else G * d
     vs = v.stride(0) if T > 1 else H * e
-    f = _fn("delta_rule", "br_dr_scan_pieces", [_P, _P, c_size_t, _P, c_size_t, _P, _P, _P, c_size_t, _P, _P, _P, _P] + [c_int] * 6 + [_P])
-    _check(f(_ptr(q), _ptr(k), qs, _ptr(v), vs, _ptr(decay), _ptr(out), _ptr(state), state.stride(0), _ptr(slots), _ptr(piece_cu),
-             _ptr(piece_slots), _ptr(piece_state), B, pieces, H, d, e, int(bool(silu)), _stream()), "dr_scan_pieces")
+    f = _fn("delta_rule", "br_dr_scan_pieces", [_P, _P, c_size_t, _P, c_size_t, _P, c_size_t] + [_P] * 5 + [c_size_t] + [_P] * 5 + [c_int] * 9 + [_P])
+    _check(f(_ptr(q), _ptr(k), qs, _ptr(v), vs, _ptr(gb), 2 * H, _ptr(decay), _ptr(skip), _ptr(out), _ptr(n_out), _ptr(state), state.stride(0),
+             _ptr(slots), _ptr(piece_cu), _ptr(piece_slots), _ptr(piece_state), _ptr(piece_decay), B, pieces, H, G, d, e, mode,
+             int(n_out is not None), int(bool(silu)), _stream()), "dr_scan_pieces")
 
 
 def tanh(x: torch.Tensor, out: torch.Tensor) -> None:
@@ -1120,18 +1266,19 @@ def route_sigmoid(scores: torch.Tensor, correction: Optional[torch.Tensor], chos
     _req(groups >= 1 and E % groups == 0 and (groups == 1 or (1 <= keep <= groups and keep * (E // groups) >= top)),
          f"route_sigmoid: {groups} runs of experts of which {keep} are kept cannot give {top} of {E} experts")
     f = _fn("routed_experts", "br_route_corrected", _ROUTE_ARGS)
-    _check(f(_ptr(scores), E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, int(groups), int(keep), 0, 1, float(out_scale),
+    _check(f(_ptr(scores), E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, int(groups), int(keep), 0, 0, 1, float(out_scale),
              _stream()), "route_sigmoid")
 
 
-_ROUTE_ARGS = [_P, c_int, _P, _P, _P] + [c_int] * 7 + [c_float, _P]
+_ROUTE_ARGS = [_P, c_int, _P, _P, _P] + [c_int] * 8 + [c_float, _P]
 
 
 def route_softmax(scores: torch.Tensor, correction: Optional[torch.Tensor], chosen: torch.Tensor, share: torch.Tensor, top: int,
-                  out_scale: float = 1.0) -> None:
+                  out_scale: float = 1.0, groups: int = 1, keep: int = 1) -> None:
     """scores float [T, E] (rows may be strided): s = the softmax over a row; the `top` numbers with the largest
     s + correction (ties to the lower one) into chosen int32 [T, top], their s as they are, times `out_scale`, into share
-    float [T, top]."""
+    float [T, top].  `groups` > 1: the numbers form that many runs of neighbours, a run scores its largest s + correction, and
+    only numbers of the `keep` best runs can be chosen."""
     _dev("route_softmax", correction, chosen, share)
     T, E = scores.shape
     _req(scores.is_cuda and scores.dtype == torch.float32 and scores.stride(1) == 1 and (T <= 1 or scores.stride(0) >= E),
@@ -1140,8 +1287,10 @@ def route_softmax(scores: torch.Tensor, correction: Optional[torch.Tensor], chos
     _req(chosen.dtype == torch.int32 and chosen.shape == (T, top) and share.dtype == torch.float32 and share.shape == (T, top),
          "route_softmax: chosen int32 and share float32 [T, top]")
     _req(0 < top <= min(E, 64) and E <= 512, f"route_softmax: {top} of {E} is outside the kernel's sizes (512 outputs, 64 chosen)")
+    _req(groups >= 1 and E % groups == 0 and (groups == 1 or (1 <= keep <= groups and keep * (E // groups) >= top)),
+         f"route_softmax: {groups} runs of which {keep} are kept cannot give {top} of {E}")
     f = _fn("routed_experts", "br_route_corrected", _ROUTE_ARGS)
-    _check(f(_ptr(scores), scores.stride(0) if T > 1 else E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, 1, 1, 1, 0,
+    _check(f(_ptr(scores), scores.stride(0) if T > 1 else E, _ptr(correction), _ptr(chosen), _ptr(share), T, E, top, int(groups), int(keep), 1, 1, 0,
              float(out_scale), _stream()), "route_softmax")
 
 

@@ -12,6 +12,7 @@ configuration or name.  Kinds:
 * `FeedForward`      adds its output to the residual stream
 * `InputJoin`        rewrites the residual rows from themselves and the embedding output, between
                      two entries of the run order
+* `Connection`       couples a half of a layer to a residual kept as several streams
 * block arrangements functions that run one layer's parts in order
 
 Tensors: the residual stream `x` is float32 `[T, hidden]` in both precisions; `h` is the
@@ -105,6 +106,11 @@ class Norm(Part):
         when the norm is not of that family."""
         return None
 
+    def point_args(self):
+        """(alpha, weight, bias) of a norm that works element by element, tanh(alpha x) weight + bias, for a kernel that
+        applies it to rows it makes; None when the norm is not of that family."""
+        return None
+
     def prepare_in_product(self, a: torch.Tensor, w: torch.Tensor, x: torch.Tensor, ws) -> Any:
         """x += a @ w^T with this norm of the new x prepared in the same kernel, if the norm
         has such a kernel for these sizes and types: returns what `product_of_prepared`
@@ -145,6 +151,9 @@ class ResidualSink:
         # `overwrite`: the rows are a branch's own output, not the residual rows: a product "added" to
         # them is stored (an arrangement that norms a branch's output before the sum hands such a sink)
         self.x, self.next_norm, self.prepared, self.overwrite = x, next_norm, None, overwrite
+        # `takes_bias`: whoever reads the rows next can add a vector to them in passing; a part whose last projection has
+        # a bias then leaves it in `bias` (float [width]) instead of launching a kernel for it
+        self.takes_bias, self.bias = False, None
 
 
 class NormedInput:
@@ -245,6 +254,21 @@ class InputJoin(Part):
         raise NotImplementedError
 
 
+class Connection(Part):
+    """Couples a half of a layer to a residual of several streams, float rows [T, streams * width]."""
+
+    def open(self, X: torch.Tensor, norm: Optional["Norm"], h: torch.Tensor, ws) -> None:
+        """h = norm of what the half reads of the streams."""
+        raise NotImplementedError
+
+    def join(self, X: torch.Tensor, branches, then: Optional["Connection"], then_norm: Optional["Norm"],
+             then_h: Optional[torch.Tensor]) -> bool:
+        """The half's output, the sum over `branches` (rows [T, width], bias or None, scale), into the streams in place.  With
+        `then`, `then_norm` and `then_h` (the next half's) it may also leave then_h as `then.open` would; returns whether
+        it did."""
+        raise NotImplementedError
+
+
 class Embedding(Part):
     def forward(self, tokens: torch.Tensor, out: torch.Tensor) -> None:
         raise NotImplementedError
@@ -257,7 +281,7 @@ class OutputHead(Part):
 
 # ------------------------------------------------------------------ registries ------
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Any]]] = {
-    "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "embedding": {}, "lm_head": {}, "input_join": {}, "block": {},
+    "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "embedding": {}, "lm_head": {}, "input_join": {}, "connection": {}, "block": {},
 }
 
 

@@ -17,6 +17,7 @@ a probe (names as the reference's tracer, crates/braidinfer-runtime/src/tracer.r
 """
 from __future__ import annotations
 
+from .. import kernels as K
 from .base import NormedInput, ResidualSink, register_part
 
 
@@ -182,6 +183,72 @@ class PrenormSideBySide:
             step.probe(f"L{step.schedule_index}.post_ffn", x)
 
 
+class HyperConnected:
+    """A residual of several streams (`ModelSpec.streams`): each half (role "mixer", then "feed_forward") reads
+    norm(u) with u what its connection (`layer.connections`) takes from the streams, and the connection writes its output
+    back into them.  Several mixers side by side (`layer.mixer` and `layer.more_mixers`, at most two) read the same rows; their
+    outputs join as a weighted sum (the connection's `branch_scales`, in that order).  Every part stores its output in float
+    rows of its own; writing them into the streams, what the next half (or the next layer's first) reads of the new
+    streams and its norm are one kernel where the norm works element by element."""
+
+    takes_streams = True
+
+    def opening(self, layer):
+        role = "mixer" if layer.mixer is not None else "feed_forward"
+        return (layer.connections[role], layer.norms.get(role)) if role in layer.connections else None
+
+    def first_norm(self, layer):
+        return None
+
+    def run(self, layer, X, step, mixer_ctx) -> None:
+        after = step.next_layer.opening() if step.next_layer is not None else None
+        halves = []
+        if layer.mixer is not None:
+            halves.append(("mixer", [(layer.mixer, (mixer_ctx,))] +
+                           [(m, (mixer_ctx.others[role],)) for role, m in layer.more_mixers.items()]))
+        if layer.feed_forward is not None:
+            halves.append(("feed_forward", [(layer.feed_forward, ())]))
+        for i, (role, parts) in enumerate(halves):
+            then = after
+            if i + 1 < len(halves):
+                nxt = halves[i + 1][0]
+                then = (layer.connections[nxt], layer.norms.get(nxt))
+            self.half(layer.connections[role], layer.norms.get(role), parts, then, X, step, layer.rt.dtype)
+            if step.probe is not None and role == "mixer":
+                self.probe(step, "post_mixer", X, layer.connections[role].width)
+        if step.probe is not None:
+            self.probe(step, "post_ffn", X, X.shape[1] if not halves else layer.connections[halves[0][0]].width)
+
+    @staticmethod
+    def probe(step, where, X, width) -> None:
+        """The sum of the streams is what stands for the residual rows."""
+        total = step.ws.get("streams_probe", (X.shape[0], width), X.dtype)
+        K.streams_open(X, total, X.shape[1] // width)
+        step.probe(f"L{step.schedule_index}.{where}", total)
+
+    @staticmethod
+    def half(connection, norm, parts, then, X, step, dtype) -> None:
+        T, W = X.shape[0], connection.width
+        prepared, step.prepared_norm = step.prepared_norm, None
+        h = step.ws.get("block_h", (T, W), dtype)
+        if not (prepared is not None and prepared[0] is connection and prepared[1] is X):
+            connection.open(X, norm, h, step.ws)
+        branches = []
+        for n, (part, extra) in enumerate(parts):
+            sink = ResidualSink(step.ws.get("branch_out" if n == 0 else f"branch_out{n}", (T, W), X.dtype), None, overwrite=True)
+            sink.takes_bias = True
+            if part.through_linear_only or part.stores_output:
+                part.forward(h, sink, step, *extra)
+            else:
+                sink.x.zero_()
+                part.forward(h, sink.x, step, *extra)
+            branches.append((sink.x, sink.bias))
+        # the halves before have read their rows by then (stream order): the next half's take the same buffer
+        if connection.join(X, branches, then[0] if then else None, then[1] if then else None, h if then else None):
+            step.prepared_norm = (then[0], X, ("connected", h))
+
+
+register_part("block", "hyper_connected", HyperConnected, replace=True)
 register_part("block", "prenorm_residual", PrenormResidual, replace=True)
 register_part("block", "prenorm_side_by_side", PrenormSideBySide, replace=True)
 register_part("block", "parallel_residual", ParallelResidual, replace=True)

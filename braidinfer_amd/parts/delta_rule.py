@@ -9,7 +9,10 @@ beta = sigmoid(W_b n) and g = exp(-exp(A_log) * softplus(W_a n + dt_bias)), one 
     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
 
 in this order (the read-out sees the token's own write).  Every head's o is divided by its root mean square over e,
-multiplied by a weight [e] shared by the heads and by silu(W_g n) [H, e], and projected by W_o.
+multiplied by a weight [e] shared by the heads and by silu(W_g n) [H, e], and projected by W_o.  With `decay_rank` there is
+one decay a head and key channel instead, diag(g) S with g = exp(-exp(A_log) * softplus(W_a2 (W_a1 n) + dt_bias)) [H, d],
+through a low-rank projection of that inner width; `gate_rank` makes the gate's projection low-rank too, W_g2 (W_g1 n), and
+`gate` "sigmoid" its activation.
 
 Lightning attention (linear attention with a fixed decay per head): q = silu(W_q n), k = silu(W_k n) (H heads of d),
 v = silu(W_v n) (H of e); S <- decay_h S + k v^T, o = S^T q, no other scale.  The concatenated heads are RMS-normed
@@ -37,12 +40,13 @@ from ..errors import ConfigError, StepError
 from ..weights import TensorSpec
 from .base import Mixer, MixerContext, RotaryTables, Runtime, register_part
 from .gated_recurrence import HGRN2, pieces_for
-from .linear import fused_layout, linear, stream_layout
+from .linear import fused_layout, linear, padded_rows, stream_layout
 
 
-def _floats(shape) -> int:
+def state_floats(heads: int, d: int, e: int) -> int:
+    """Floats of a sequence's [d, e] states as the scan kernels keep them."""
     n = 1
-    for s in shape:
+    for s in K.glr_state_shape(heads, d, e):
         n *= int(s)
     return n
 
@@ -52,10 +56,15 @@ class GatedDeltaRule(Mixer):
     through_linear_only = True
 
     NAMES = {"q": "q", "k": "k", "v": "v", "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv", "b": "b", "a": "a",
-             "A_log": "A_log", "dt_bias": "dt_bias", "norm": "norm", "g": "g", "o": "o"}
+             "a1": "a1", "a2": "a2", "g1": "g1", "g2": "g2", "A_log": "A_log", "dt_bias": "dt_bias", "norm": "norm", "g": "g", "o": "o"}
 
     def __init__(self, hidden_size: int, num_heads: int, num_key_heads: int, key_dim: int, value_dim: int, taps: int,
-                 norm_eps: float, out_scale: float = 1.0, names: Optional[Dict[str, str]] = None):
+                 norm_eps: float, out_scale: float = 1.0, names: Optional[Dict[str, str]] = None, decay_rank: Optional[int] = None,
+                 gate_rank: Optional[int] = None, gate: str = "silu"):
+        if any(r is not None and int(r) <= 0 for r in (decay_rank, gate_rank)) or gate not in ("silu", "sigmoid") or \
+                (gate_rank is not None and decay_rank is None):
+            raise ConfigError(f"delta rule: inner widths {decay_rank} of the decays and {gate_rank} of the gate must be positive where given (a "
+                              f"low-rank gate goes with low-rank decays), the gate 'silu' or 'sigmoid', got {gate!r}")
         if num_heads <= 0 or num_key_heads <= 0 or num_heads % num_key_heads:
             raise ConfigError(f"delta rule: {num_heads} heads are not a multiple of {num_key_heads} key heads")
         if not 0 < key_dim <= 512 or not 0 < value_dim <= 512 or not 1 <= int(taps) <= 16:
@@ -65,7 +74,11 @@ class GatedDeltaRule(Mixer):
         self.taps, self.eps, self.out_scale = int(taps), float(norm_eps), float(out_scale)
         self.names = dict(self.NAMES, **(names or {}))
         self.C = 2 * self.ng * self.d + self.nh * self.e          # convolved channels: q | k | v
-        self.state_floats = _floats(K.glr_state_shape(self.nh, self.d, self.e))
+        self.state_floats = state_floats(self.nh, self.d, self.e)
+        self.decay_rank = None if decay_rank is None else int(decay_rank)
+        self.gate_rank = None if gate_rank is None else int(gate_rank)
+        self.gate_sigmoid = gate == "sigmoid"
+        self.w_low = None
         self.w_in = self.w_o = self.conv = self.conv_t = self.a_log = self.dt_bias = self.norm_w = None
 
     def weight_specs(self, prefix: str) -> List[TensorSpec]:
@@ -78,17 +91,27 @@ class GatedDeltaRule(Mixer):
                 TensorSpec(prefix + n["v_conv"], (he, self.taps), kind="vector", init="normal"),
                 TensorSpec(prefix + n["b"], (self.nh, self.H)),
                 TensorSpec(prefix + n["A_log"], (self.nh,), kind="vector", init="normal"),
-                TensorSpec(prefix + n["norm"], (self.e,), kind="vector", init="ones"),
-                TensorSpec(prefix + n["a"], (self.nh, self.H)),
-                TensorSpec(prefix + n["dt_bias"], (self.nh,), kind="vector", init="normal"),
-                TensorSpec(prefix + n["g"], (he, self.H)),
-                TensorSpec(prefix + n["o"], (self.H, he))]
+                TensorSpec(prefix + n["norm"], (self.e,), kind="vector", init="ones")] + \
+               ([TensorSpec(prefix + n["a"], (self.nh, self.H))] if self.decay_rank is None else
+                [TensorSpec(prefix + n["a1"], (self.decay_rank, self.H)), TensorSpec(prefix + n["a2"], (self.nh * self.d, self.decay_rank))]) + \
+               [TensorSpec(prefix + n["dt_bias"], (self.nh * (1 if self.decay_rank is None else self.d),), kind="vector", init="normal")] + \
+               ([TensorSpec(prefix + n["g"], (he, self.H))] if self.gate_rank is None else
+                [TensorSpec(prefix + n["g1"], (self.gate_rank, self.H)), TensorSpec(prefix + n["g2"], (he, self.gate_rank))]) + \
+               [TensorSpec(prefix + n["o"], (self.H, he))]
 
     def load(self, tensors: Dict[str, torch.Tensor], prefix: str, rt: Runtime) -> None:
         self.rt = rt
         n = self.names
-        # one product: q | k | v | b | a | g
-        self.w_in = fused_layout([tensors[prefix + n[x]] for x in ("q", "k", "v", "b", "a", "g")], rt)
+        # one product: q | k | v | b | a | g, or with low-rank projections q | k | v | b | (g |) a1 (| g1)
+        if self.decay_rank is None:
+            first = ("q", "k", "v", "b", "a", "g")
+        elif self.gate_rank is None:
+            first = ("q", "k", "v", "b", "g", "a1")
+        else:
+            first = ("q", "k", "v", "b", "a1", "g1")
+        self.w_in = fused_layout([tensors[prefix + n[x]] for x in first], rt)
+        if self.decay_rank is not None:
+            self._load_low(tensors, prefix, rt)
         self.w_o = stream_layout(tensors[prefix + n["o"]], rt)
         self.conv = rt.own(torch.cat([tensors[prefix + n[x]].to(torch.float32).reshape(-1, self.taps)
                                       for x in ("q_conv", "k_conv", "v_conv")]))
@@ -98,6 +121,21 @@ class GatedDeltaRule(Mixer):
         # the head norm's weight for every head, with the mixer's multiplier
         self.norm_w = rt.own((tensors[prefix + n["norm"]].to(torch.float32).reshape(-1) * self.out_scale).repeat(self.nh))
 
+    def _load_low(self, tensors, prefix: str, rt: Runtime) -> None:
+        """The second matrices of the low-rank projections.  Two of them are one product over both inner rows side by side:
+        W_a2 and W_g2 stand on the diagonal of a matrix of zeros."""
+        n, ra, rg = self.names, self.decay_rank, self.gate_rank or 0
+        a2 = tensors[prefix + n["a2"]]
+        if not rg:
+            self.w_low = stream_layout(a2, rt)
+            return
+        g2 = tensors[prefix + n["g2"]]
+        w = rt.empty((self.nh * (self.d + self.e), ra + rg), torch.float32 if torch.float32 in (a2.dtype, g2.dtype) else a2.dtype)
+        w.zero_()
+        w[:self.nh * self.d, :ra].copy_(a2)
+        w[self.nh * self.d:, ra:].copy_(g2)
+        self.w_low = w
+
     def state_need(self) -> StateNeed:
         # the heads' states as the scan keeps them, then the convolution's last inputs [taps - 1][channels]
         return StateNeed((self.state_floats + (self.taps - 1) * self.C,), torch.float32)
@@ -106,20 +144,31 @@ class GatedDeltaRule(Mixer):
         T, nh, ng, d, e, C = step.n_tokens, self.nh, self.ng, self.d, self.e, self.C
         if ctx.state is None:
             raise StepError("delta rule: the cache gave this mixer no state")
-        rows = step.ws.get("dr_rows", (T, C + 2 * nh + nh * e), torch.float32)
+        low_rank = self.decay_rank is not None
+        width = C + (2 * nh + nh * e if not low_rank else nh + self.decay_rank + (self.gate_rank or nh * e))
+        rows = padded_rows(step.ws, "dr_rows", T, width)
         linear(h, self.w_in, rows, step.ws)
+        decay = gc = None
+        if not low_rank:
+            gate = rows[:, C + 2 * nh:]
+        else:
+            n_low = self.decay_rank + (self.gate_rank or 0)
+            second = step.ws.get("dr_low", (T, nh * d + (nh * e if self.gate_rank else 0)), torch.float32)
+            linear(rows[:, width - n_low:], self.w_low, second, step.ws)
+            decay, gate = second[:, :nh * d], (second[:, nh * d:] if self.gate_rank else rows[:, C + nh:C + nh + nh * e])
+            gc = step.ws.get("dr_gc", (T, nh * d), torch.float32)
         q = step.ws.get("dr_q", (T, ng * d), torch.float32)
         k = step.ws.get("dr_k", (T, ng * d), torch.float32)
         v = step.ws.get("dr_v", (T, nh * e), torch.float32)
         gb = step.ws.get("dr_gb", (T, 2 * nh), torch.float32)
         kept = ctx.state[:, self.state_floats:] if self.taps > 1 else None
         K.dr_conv_prepare(rows, self.conv, kept, self.a_log, self.dt_bias, step.seq_of_token, step.cu_seqlens, step.slots,
-                          q, k, v, gb, step.n_seqs, ng, nh, d, e, taps_t=self.conv_t)
+                          q, k, v, gb, step.n_seqs, ng, nh, d, e, taps_t=self.conv_t, decay=decay, gc=gc, single_tokens=step.is_decode)
         o = step.ws.get("dr_o", (T, nh * e), torch.float32)
         S = ctx.state[:, :self.state_floats].view((-1,) + tuple(K.glr_state_shape(nh, d, e)))
-        K.dr_scan(q, k, v, gb, None, o, S, step.cu_seqlens, step.slots, step.n_seqs, nh, ng, d, e)
+        K.dr_scan(q, k, v, gb, None, o, S, step.cu_seqlens, step.slots, step.n_seqs, nh, ng, d, e, gc=gc)
         y = step.ws.get("dr_y", (T, nh * e), self.rt.dtype)
-        K.head_norm_gate(o, self.norm_w, rows[:, C + 2 * nh:], y, nh, e, self.eps)
+        K.head_norm_gate(o, self.norm_w, gate, y, nh, e, self.eps, gate_sigmoid=self.gate_sigmoid)
         linear(y, self.w_o, x, step.ws, accumulate=True)
 
 

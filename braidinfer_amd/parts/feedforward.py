@@ -14,7 +14,7 @@ with an expert W_d (silu(W_g n) * (W_u n)) without biases.  `scoring` "sigmoid" 
 the choice is made on s + a learnt correction per expert, among the experts of the best `groups_keep` of `groups`
 equal runs of neighbouring experts (a run scores the sum of its two largest corrected scores); the shares are the
 chosen experts' s over their sum.  `scoring` "softmax_all": s is the softmax over all outputs, the choice is made on s + a
-learnt correction, and the shares are the chosen s as they are.  `shared_size` adds a gated unit of that inner width
+learnt correction, and the shares are the chosen s as they are; `correction` False: there is none.  With that scoring a run of experts scores its largest s.  `shared_size` adds a gated unit of that inner width
 that every token passes; `shared_gate` multiplies it by the sigmoid of a learnt product of the token, one number.
 `limit`, `alpha`: the experts (`shared_limit`: the shared unit) are clamped gated units without biases.  `identity` adds
 that many outputs behind the experts' whose "expert" returns its input row and has no matrices.  The reference has none
@@ -138,7 +138,7 @@ class RoutedExperts(FeedForward):
                  names: Optional[Dict[str, str]] = None, out_scale: float = 1.0, scoring: str = "softmax",
                  groups: int = 1, groups_keep: int = 1, shared_size: int = 0, identity: int = 0,
                  limit: Optional[float] = None, alpha: float = 1.702, shared_limit: Optional[float] = None,
-                 shared_gate: bool = False):
+                 shared_gate: bool = False, correction: bool = True):
         """`names`: "expert" with {e} for the expert's number (the prefix of its three matrices "gate", "up", "down"),
         "router", "router_bias", "correction", "shared" (the prefix of the shared unit's), "shared_gate".  `limit` None: the
         experts are silu units, else clamped ones (`shared_limit`, None: the same, for the shared unit).  `out_scale` multiplies what is added to the residual rows (it rides on the shares)."""
@@ -159,10 +159,10 @@ class RoutedExperts(FeedForward):
         if limit is not None and not (self.limit > 0 and self.alpha > 0) or (shared_limit is not None and not float(shared_limit) > 0):
             raise ConfigError(f"routed experts: the clamped units' limits ({limit}, {shared_limit}) and factor ({alpha}) must be positive")
         self.groups, self.groups_keep, self.shared_size = int(groups), int(groups_keep), int(shared_size or 0)
-        if self.groups < 1 or self.E % self.groups or (self.groups > 1 and not self.sigmoid) or self.shared_size < 0 or \
+        if self.groups < 1 or self.E % self.groups or (self.groups > 1 and (self.identity or not (self.sigmoid or self.softmax_all))) or self.shared_size < 0 or \
                 (self.groups > 1 and not (1 <= self.groups_keep <= self.groups and self.groups_keep * (self.E // self.groups) >= self.top)):
             raise ConfigError(f"routed experts: {groups} runs of experts of which {groups_keep} are kept must divide the "
-                              f"{num_experts} experts (sigmoid scoring) and leave {top} to choose")
+                              f"{num_experts} experts (sigmoid or softmax_all scoring, no identities) and leave {top} to choose")
         self.router_bias = bool(router_bias) and not self.sigmoid and not self.softmax_all
         self.shared_gate = bool(shared_gate) and self.shared_size > 0
         self.names = dict({"expert": "e{e}.", "gate": "gate", "up": "up", "down": "down", "router": "router",
@@ -178,7 +178,7 @@ class RoutedExperts(FeedForward):
             else:
                 self.shared = ClampedGLU(self.H, self.shared_size, self.limit if shared_limit is None else float(shared_limit), self.alpha,
                                          names=sh, bias=False)
-        self.correction = None
+        self.corrected, self.correction = bool(correction) and (self.sigmoid or self.softmax_all), None
         self.w_gu = self.w_down = self.w_router = self.b_router = None
 
     def _expert(self, prefix: str, e: int, what: str) -> str:
@@ -193,7 +193,7 @@ class RoutedExperts(FeedForward):
         out.append(TensorSpec(prefix + self.names["router"], (self.n_out, self.H)))
         if self.router_bias:
             out.append(TensorSpec(prefix + self.names["router_bias"], (self.E,), kind="vector", init="normal"))
-        if self.sigmoid or self.softmax_all:
+        if self.corrected:
             out.append(TensorSpec(prefix + self.names["correction"], (self.n_out,), kind="vector", init="normal"))
         if self.shared is not None:
             out += self.shared.weight_specs(prefix)
@@ -224,7 +224,7 @@ class RoutedExperts(FeedForward):
         self.w_router = rt.own(router)
         if self.router_bias:
             self.b_router = rt.own(tensors[prefix + self.names["router_bias"]].to(torch.float32).reshape(-1))
-        if self.sigmoid or self.softmax_all:
+        if self.corrected:
             self.correction = rt.own(tensors[prefix + self.names["correction"]].to(torch.float32).reshape(-1))
         if self.shared is not None:
             self.shared.load(tensors, prefix, rt)
@@ -253,7 +253,7 @@ class RoutedExperts(FeedForward):
         chosen = step.ws.get("moe_chosen", (T, self.top), torch.int32)
         share = step.ws.get("moe_share", (T, self.top), torch.float32)
         if self.softmax_all:
-            K.route_softmax(scores[:, :self.n_out], self.correction, chosen, share, self.top, self.out_scale)
+            K.route_softmax(scores[:, :self.n_out], self.correction, chosen, share, self.top, self.out_scale, self.groups, self.groups_keep)
         elif self.sigmoid:
             K.route_sigmoid(scores, self.correction, chosen, share, self.top, self.groups, self.groups_keep, self.out_scale)
         else:

@@ -55,7 +55,10 @@ def linear(a, w: torch.Tensor, out, ws, accumulate: bool = False) -> None:
         return
     if w.dtype == torch.bfloat16 and a.dtype == torch.float32:
         a16 = ws.get("linear_in16", a.shape, torch.bfloat16)
-        K.convert(a.contiguous(), a16)
+        if a.is_contiguous():
+            K.convert(a, a16)
+        else:                              # a column range of wider rows
+            K.rows_into(a, a16)
         linear(a16, w, out, ws, accumulate)
         return
     raise TypeError(f"linear: activations {a.dtype}, weight {w.dtype}")
@@ -77,6 +80,11 @@ def linear_runs(a, w: torch.Tensor, n_out: int, ws):
     scratch = ws.get("gemm_scratch", (K.GEMM_SCRATCH_FLOATS,), torch.float32)
     runs = K.gemm_wide_partial(a, w, n_out, scratch)
     return ProductRuns(scratch, runs, a.shape[0], n_out) if runs else None
+
+
+def padded_rows(ws, name: str, T: int, width: int) -> torch.Tensor:
+    """Float rows [T, width] whose starts lie at multiples of 16 bytes."""
+    return ws.get(name, (T, -(-width // 4) * 4), torch.float32)[:, :width]
 
 
 BLOCK_FROM_ROWS = 8192

@@ -14,6 +14,9 @@ checkpoints the reference loads; "" where the prefix is the whole name).
 (a design that norms a half's output only).  It has no weights; a norm that adds behind the half before can leave
 these rows in the same kernel, as it would leave a following norm's.
 
+`dynamic_tanh`: y = tanh(alpha x) * w + b element by element, with a learnt scalar alpha: no statistics at all, so a
+kernel that makes x can apply it in passing (`point_args`).
+
 `layer_scale`: no norm either, y = x * w channel by channel with a learnt vector: what stands behind a half whose output
 is scaled before it joins the residual rows."""
 from __future__ import annotations
@@ -170,6 +173,36 @@ class LayerScale(Norm):
         return nxt is not None
 
 
+class DynamicTanh(Norm):
+    """tanh(alpha x) w + b; the scalar and the bias are named behind the weight (`<weight>.alpha`, `<weight>.b`)."""
+
+    graph_safe = True
+
+    def __init__(self, size: int, tensor: str = "weight"):
+        self.size, self.tensor = int(size), tensor
+        self.weight = self.bias = self.alpha = None
+
+    def weight_specs(self, prefix: str) -> List[TensorSpec]:
+        n = prefix + self.tensor
+        return [TensorSpec(n, (self.size,), kind="vector", init="ones"), TensorSpec(n + ".b", (self.size,), kind="vector", init="normal"),
+                TensorSpec(n + ".alpha", (), kind="vector", init="ones")]
+
+    def load(self, tensors: Dict[str, torch.Tensor], prefix: str, rt: Runtime) -> None:
+        self.rt = rt
+        n = prefix + self.tensor
+        self.weight = rt.own(tensors[n].to(torch.float32).reshape(-1))
+        self.bias = rt.own(tensors[n + ".b"].to(torch.float32).reshape(-1))
+        self.alpha = rt.own(tensors[n + ".alpha"].to(torch.float32).reshape(1))
+
+    def point_args(self):
+        return self.alpha, self.weight, self.bias
+
+    def forward(self, x, out, rows=None):
+        K.streams_open(x, out, 1, norm=self.point_args(), rows=rows)
+        return out
+
+
+register_part("norm", "dynamic_tanh", DynamicTanh, replace=True)
 register_part("norm", "layer_scale", LayerScale, replace=True)
 register_part("norm", "rows", PlainRows, replace=True)
 register_part("norm", "rmsnorm", RMSNorm, replace=True)

@@ -18,7 +18,7 @@ by a temperature that grows with the logarithm of the position, 1 + c ln(floor((
 the heads' outputs may pass a sigmoid gate projected from the mixer's input, one number per output element or one
 per head (`gate` "element" / "head"), before the output projection; a learnt factor per head may multiply its scores
 (`head_temp`: it rides on the queries); every head's value may be divided by its root mean square over the head, without
-a weight, before it is stored (`v_norm_eps`); the rotation's pairs are the encoding's, (i, i + dims/2) or neighbours; `out_scale` multiplies what the mixer adds to the
+a weight, before it is stored (`v_norm_eps`); the rotation's pairs are the encoding's, (i, i + dims/2) or neighbours; `out_bias` adds a bias behind the output projection; `out_scale` multiplies what the mixer adds to the
 residual rows (it rides on the gate, or on the output matrix where there is none).
 
 Further rules of what a query sees, each a parameter: `chunk` C cuts the sequence into runs of C positions counted
@@ -52,7 +52,7 @@ from .. import kernels as K
 from ..cache import CacheNeed
 from ..errors import ConfigError, StepError
 from ..weights import TensorSpec
-from .base import Mixer, MixerContext, RotaryTables, Runtime, register_part
+from .base import Mixer, MixerContext, ResidualSink, RotaryTables, Runtime, register_part
 from .linear import fused_layout, linear, stream_layout
 
 MAX_WIDTH = 512      # of a head's keys or values: the kernels' limit
@@ -82,7 +82,7 @@ class PooledWindowAttention(Mixer):
 
     NO_WINDOW = 1 << 30          # the kernels' window when every earlier token is seen: beyond any position
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "gate": "g_proj.weight",
-             "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
+             "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
              "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "value_mix": "value_mix", "sink": "sink",
              "head_temp": "temp", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
 
@@ -94,7 +94,7 @@ class PooledWindowAttention(Mixer):
                  q_temp=None, gate: Optional[str] = None, out_scale: float = 1.0, chunk: Optional[int] = None,
                  keep_first: int = 0, softcap: Optional[float] = None, qk_norm_over: str = "head", maps: int = 1,
                  diff: Optional[float] = None, head_norm_eps: Optional[float] = None, head_temp: bool = False,
-                 v_norm_eps: Optional[float] = None):
+                 v_norm_eps: Optional[float] = None, out_bias: bool = False):
         """`qk_norm_eps` None: no query/key norm.  `value_mix`: None, "source" (this layer's values are what
         later layers of the same `value_mix_group` mix with; its own scalar is loaded and unused) or "mix"."""
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
@@ -144,6 +144,7 @@ class PooledWindowAttention(Mixer):
         self.kw = self.maps * self.dk          # a key row of the cache, and a query row the kernels see
         self.head_temp, self.temps = bool(head_temp), None
         self.v_norm_eps = None if v_norm_eps is None else float(v_norm_eps)
+        self.out_bias, self.b_o = bool(out_bias), None
         self.adjacent = False                  # the encoding's pairs; set by check_positions
         self.sinks = None
         self.pair_factor = 0.0
@@ -183,6 +184,8 @@ class PooledWindowAttention(Mixer):
         if self.value_mix is not None:
             out.append(TensorSpec(prefix + n["value_mix"], (), kind="vector", init="normal"))
         out.append(TensorSpec(prefix + n["o"], (self.H, self.nq * self.dv)))
+        if self.out_bias:
+            out.append(TensorSpec(prefix + n["o_bias"], (self.H,), kind="vector", init="normal"))
         return out
 
     def load(self, tensors: Dict[str, torch.Tensor], prefix: str, rt: Runtime) -> None:
@@ -196,6 +199,8 @@ class PooledWindowAttention(Mixer):
         if self.gate is None and self.out_scale != 1.0:          # no gate to carry the multiplier: the matrix does
             w_o = (w_o.to(torch.float32) * self.out_scale).to(w_o.dtype)
         self.w_o = stream_layout(w_o, rt)
+        if self.out_bias:
+            self.b_o = rt.own(tensors[prefix + n["o_bias"]].to(torch.float32).reshape(-1) * self.out_scale)
         if self.bias:
             self.b_qkv = rt.own(torch.cat([tensors[prefix + n[x]].to(torch.float32).reshape(-1) for x in ("q_bias", "k_bias", "v_bias")]))
         if self.qk_norm_eps is not None and self.qk_norm_weights:
@@ -314,7 +319,15 @@ class PooledWindowAttention(Mixer):
             K.pwa_pair_combine(o2, o, nq, dv, self.pair_factor, self.head_norm_eps, (1.0 - self.diff) * self.out_scale)
         if self.gate is not None:
             K.pwa_gate(o, qkv[:, self.gate_col0:], nq, dv, self.gate == "head", self.out_scale)
+        if self.out_bias and isinstance(x, ResidualSink):
+            # the reader of the rows adds the bias where it can; no norm is prepared from sums that still lack it
+            if x.takes_bias:
+                x.bias = self.b_o
+            else:
+                x.next_norm = None
         linear(o, self.w_o, x, step.ws, accumulate=True)
+        if self.out_bias and not (isinstance(x, ResidualSink) and x.takes_bias):
+            K.add_bias_rows(x.x if isinstance(x, ResidualSink) else x, self.b_o)
 
 
 register_part("mixer", "pooled_window_attention", PooledWindowAttention, replace=True)
