@@ -76,7 +76,7 @@ LAUNCHERS = ["embedding", "rmsnorm", "layernorm", "scale_", "rope_table", "rope_
              "latent_prepare", "head_linear", "route_topk", "experts_up", "experts_down", "experts_sort", "experts_gather",
              "experts_combine", "experts_up_grouped", "experts_down_grouped", "experts_gemm", "clamped_glu", "add_bias_rows",
              "add_position_rows", "pwa_gate", "dr_conv_prepare", "dr_scan", "dr_scan_pieces", "silu_rows", "pwa_pair_combine",
-             "route_sigmoid", "dr_rotate_rows", "route_softmax", "rows_into"]
+             "route_sigmoid", "dr_rotate_rows", "route_softmax", "rows_into", "streams_spread", "streams_open", "streams_join", "ssm_prepare", "exp_gates"]
 
 
 def kernel_share(torch, eng, entries_of, classes):
@@ -271,7 +271,10 @@ class Shape:
 # same kernels, a decayed sum of key-value products per head, routed experts) at equal width and number of layer runs.
 # `--design finosun`: the Finosun design beside Ladadra (the library's closest model: window attention with a norm over
 # the projection, halves that pass a vector behind them, corrected routed experts with a shared one), likewise.
+# `--design tuzisun`: the Tuzisun design beside Zivovik (the library's closest model: attention and a delta rule side by
+# side on one input, a decayed outer sum, routed experts), likewise.
 DESIGN_SIZES = {
+    "tuzisun": {"1b": ("tuzisun-1b", "zivovik-1b"), "7b": ("tuzisun-7b", "zivovik-7b")},
     "finosun": {"1b": ("finosun-1b", "ladadra-1b"), "7b": ("finosun-7b", "ladadra-7b")},
     "ladadra": {"1b": ("ladadra-1b", "zivovik-1b"), "7b": ("ladadra-7b", "zivovik-7b")},
     "zivovik": {"1b": ("zivovik-1b", "sidirax-1b"), "7b": ("zivovik-7b", "sidirax-7b")},
@@ -404,7 +407,8 @@ def design_comparison(args) -> int:
     import torch
     import braidinfer_amd as B
     sizes = DESIGN_SIZES[args.design]
-    beside = {"sidirax": "kesitar", "zivovik": "sidirax", "ladadra": "zivovik", "finosun": "ladadra"}.get(args.design, "mistral")
+    beside = {"sidirax": "kesitar", "zivovik": "sidirax", "ladadra": "zivovik", "finosun": "ladadra",
+              "tuzisun": "zivovik"}.get(args.design, "mistral")
     line = {"metric": f"{args.design} beside {beside} at equal size: prefill and decode tokens/s, bf16, random weights",
             "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "layers": args.layers or 8,
             "steps": args.steps, "warmup": args.warmup, "sizes": {}}

@@ -354,18 +354,21 @@ extern "C" int br_ssm_prepare(const float* x, size_t width, const float* taps_t,
 // Per head the logarithms of an input and a forget gate from their float sums, i = cap tanh((zi + bi) / cap) and
 // f = log sigmoid(cap tanh((zf + bf) / cap)), and the running maximum m_t = max(f_t + m_(t-1), i_t) that a memory of
 // exponential gates is kept relative to (a slot keeps the last m; 0 in a new one).  gb [T, 2 H] takes
-// exp(f_t + m_(t-1) - m_t), then exp(i_t - m_t); m [T, H] the maxima.  Tokens are taken 64 at a time, one a lane: m is a
-// prefix of the maps m -> max(m + a, b), composed across the wave.  grid (B, H), one wave.
-__global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__ zi, const float* __restrict__ zf, size_t stride,
-                                                       const float* __restrict__ bi, const float* __restrict__ bf, float cap,
-                                                       float* kept, size_t kept_stride, const int* __restrict__ cu_seqlens,
-                                                       const int* __restrict__ slots, float* __restrict__ gb, float* __restrict__ m_out,
-                                                       int H) {
-    const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+// exp(f_t + m_(t-1) - m_t), then exp(i_t - m_t); m [T, H] the maxima.  m is a prefix of the maps m -> max(m + a, b), one a
+// token: composed across a wave's 64 tokens and, in long steps, across the WAVES waves of a workgroup (64 tokens each at a
+// time) through LDS.  grid (B, H), 64 WAVES threads.
+template <int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void exp_gates_kernel(const float* __restrict__ zi, const float* __restrict__ zf, size_t stride,
+                                                               const float* __restrict__ bi, const float* __restrict__ bf, float cap,
+                                                               float* kept, size_t kept_stride, const int* __restrict__ cu_seqlens,
+                                                               const int* __restrict__ slots, float* __restrict__ gb,
+                                                               float* __restrict__ m_out, int H) {
+    __shared__ float wa[WAVES], wb[WAVES];
+    const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int slot = slots[b], t0 = cu_seqlens[b], t1 = cu_seqlens[b + 1];
     float m0 = slot >= 0 ? kept[(size_t)slot * kept_stride + h] : 0.f;
-    for (int tc = t0; tc < t1; tc += 64) {
-        const int t = tc + lane;
+    for (int tc = t0; tc < t1; tc += 64 * WAVES) {
+        const int t = tc + (int)threadIdx.x;
         const bool on = t < t1;
         float i = -INFINITY, f = 0.f;
         if (on) {
@@ -373,105 +376,45 @@ __global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__
             const float z = cap * tanhf((zf[(size_t)t * stride + h] + bf[h]) / cap);
             f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
         }
-        float A = f, Bm = i;          // the map of the tokens up to this one: m -> max(m + A, Bm)
+        float A = f, Bm = i;          // the map of the wave's tokens up to this one: m -> max(m + A, Bm)
 #pragma unroll
         for (int o = 1; o < 64; o <<= 1) {
             const float pa = __shfl_up(A, o, WAVE), pb = __shfl_up(Bm, o, WAVE);
             if (lane >= o) { Bm = fmaxf(pb + A, Bm); A += pa; }
         }
-        const float m = fmaxf(m0 + A, Bm);
+        float start = m0;             // m in front of the wave's tokens
+        if (WAVES > 1) {
+            __syncthreads();
+            if (lane == 63) { wa[wave] = A; wb[wave] = Bm; }
+            __syncthreads();
+#pragma unroll
+            for (int w = 0; w < WAVES; ++w) {
+                const float behind = fmaxf(m0 + wa[w], wb[w]);
+                if (w < wave) start = behind;
+                m0 = behind;
+            }
+        }
+        const float m = fmaxf(start + A, Bm);
         float before = __shfl_up(m, 1, WAVE);
-        if (lane == 0) before = m0;
+        if (lane == 0) before = start;
         if (on) {
             gb[(size_t)t * 2 * H + h] = expf(f + before - m);
             gb[(size_t)t * 2 * H + H + h] = expf(i - m);
             m_out[(size_t)t * H + h] = m;
         }
-        m0 = __shfl(m, 63, WAVE);     // lanes behind the last token hold its m
+        if (WAVES == 1) m0 = __shfl(m, 63, WAVE);     // lanes behind the last token hold its m
     }
-    if (lane == 0 && slot >= 0) kept[(size_t)slot * kept_stride + h] = m0;
+    if (threadIdx.x == 0 && slot >= 0) kept[(size_t)slot * kept_stride + h] = m0;
 }
 
+// `single_tokens`: no sequence brings more than one token (one wave a head).
 extern "C" int br_exp_gates(const float* zi, const float* zf, size_t stride, const float* bi, const float* bf, float cap, float* kept,
                             size_t kept_stride, const int* cu_seqlens, const int* slots, float* gb, float* m_out, int B, int H,
-                            hipStream_t s) {
+                            int single_tokens, hipStream_t s) {
     if (B <= 0) return BR_OK;
     if (H <= 0 || H > 65535 || stride < (size_t)H || !(cap > 0.f) || !kept || kept_stride < (size_t)H || !bi || !bf) return BR_BAD_ARG;
-    exp_gates_kernel<<<dim3(B, H), 64, 0, s>>>(zi, zf, stride, bi, bf, cap, kept, kept_stride, cu_seqlens, slots, gb, m_out, H);
-    return br_check_launch();
-}
-
-// x[t, :n] <- silu(x[t, :n]) in place on float rows `stride` apart (projections' sums that go on as activations: done
-// once here, not by every workgroup of a scan that reads them).  VEC: four a thread, for n, stride and pointer in fours.
-template <bool VEC>
-__global__ __launch_bounds__(256) void dr_silu_rows_kernel(float* __restrict__ x, size_t stride, int n, size_t total) {
-    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= total) return;
-    if (VEC) {
-        const size_t per = (size_t)n / 4, t = i / per, c = (i - t * per) * 4;
-        f32x4* p = (f32x4*)(x + t * stride + c);
-        f32x4 v = *p;
-#pragma unroll
-        for (int k = 0; k < 4; ++k) v[k] = dr_silu(v[k]);
-        *p = v;
-    } else {
-        const size_t t = i / n, c = i - t * n;
-        float* p = x + t * stride + c;
-        *p = dr_silu(*p);
-    }
-}
-
-extern "C" int br_silu_rows(float* x, size_t stride, int T, int n, hipStream_t s) {
-    if (T <= 0 || n <= 0) return BR_OK;
-    if (stride < (size_t)n) return BR_BAD_ARG;
-    const bool vec = n % 4 == 0 && stride % 4 == 0 && ((uintptr_t)x % 16) == 0;
-    const size_t total = vec ? (size_t)T * (n / 4) : (size_t)T * n;
-    const size_t blocks = (total + 255) / 256;
-    if (blocks > 0x7fffffffULL) return BR_BAD_ARG;
-    if (vec) dr_silu_rows_kernel<true><<<(unsigned)blocks, 256, 0, s>>>(x, stride, n, total);
-    else dr_silu_rows_kernel<false><<<(unsigned)blocks, 256, 0, s>>>(x, stride, n, total);
-    return br_check_launch();
-}
-
-// q and k rows (float sums of their projections, rows `stride` apart, `heads` heads of d channels each) turned in place
-// by their tokens' positions: of the first `rd` channels of a head, channel i < rd / 2 and channel i + rd / 2 form
-// a pair that is turned by the angle whose cosine and sine are cs[t, i], sn[t, i] ((u, v) -> (u c - v s, v c + u s));
-// the other channels pass.  Every channel of q is then multiplied by `q_mul` and every channel of k by `k_mul`.
-// A thread a channel below rd / 2 (it owns the pair) or from rd on; grid over T * heads * (d - rd / 2) threads.
-__global__ __launch_bounds__(256) void dr_rotate_rows_kernel(float* __restrict__ q, float* __restrict__ k, size_t stride,
-                                                             const float* __restrict__ cs, const float* __restrict__ sn,
-                                                             int rd, int heads, int d, float q_mul, float k_mul, size_t total) {
-    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= total) return;
-    const int half = rd >> 1, per = d - half;
-    const size_t th = i / per;
-    const int j = (int)(i - th * per);
-    const size_t t = th / heads;
-    const int h = (int)(th - t * heads);
-    float* qr = q + t * stride + (size_t)h * d;
-    float* kr = k + t * stride + (size_t)h * d;
-    if (j < half) {
-        const float c = cs[t * half + j], s_ = sn[t * half + j];
-        const float qu = qr[j], qv = qr[j + half], ku = kr[j], kv = kr[j + half];
-        qr[j] = (qu * c - qv * s_) * q_mul;
-        qr[j + half] = (qv * c + qu * s_) * q_mul;
-        kr[j] = (ku * c - kv * s_) * k_mul;
-        kr[j + half] = (kv * c + ku * s_) * k_mul;
-    } else {
-        const int ch = j + half;                    // channels from rd on
-        qr[ch] *= q_mul;
-        kr[ch] *= k_mul;
-    }
-}
-
-extern "C" int br_dr_rotate_rows(float* q, float* k, size_t stride, const float* cs, const float* sn, int rd, int T, int heads,
-                                 int d, float q_mul, float k_mul, hipStream_t s) {
-    if (T <= 0) return BR_OK;
-    if (heads <= 0 || d <= 0 || rd < 0 || (rd & 1) || rd > d || stride < (size_t)heads * d || (rd > 0 && (!cs || !sn))) return BR_BAD_ARG;
-    const size_t total = (size_t)T * heads * (d - rd / 2);
-    const size_t blocks = (total + 255) / 256;
-    if (blocks > 0x7fffffffULL) return BR_BAD_ARG;
-    dr_rotate_rows_kernel<<<(unsigned)blocks, 256, 0, s>>>(q, k, stride, cs, sn, rd, heads, d, q_mul, k_mul, total);
+    if (single_tokens) exp_gates_kernel<1><<<dim3(B, H), 64, 0, s>>>(zi, zf, stride, bi, bf, cap, kept, kept_stride, cu_seqlens, slots, gb, m_out, H);
+    else exp_gates_kernel<16><<<dim3(B, H), 1024, 0, s>>>(zi, zf, stride, bi, bf, cap, kept, kept_stride, cu_seqlens, slots, gb, m_out, H);
     return br_check_launch();
 }
 

@@ -1057,10 +1057,11 @@ def ssm_prepare(x: torch.Tensor, taps_t: torch.Tensor, bias: Optional[torch.Tens
 
 
 def exp_gates(zi: torch.Tensor, zf: torch.Tensor, bi: torch.Tensor, bf: torch.Tensor, cap: float, kept: torch.Tensor,
-              cu_seqlens: torch.Tensor, slots: torch.Tensor, gb: torch.Tensor, m: torch.Tensor, B: int) -> None:
+              cu_seqlens: torch.Tensor, slots: torch.Tensor, gb: torch.Tensor, m: torch.Tensor, B: int, single_tokens: bool = False) -> None:
     """Exponential input and sigmoid forget gates over a running maximum: i = cap tanh((zi + bi) / cap),
     f = log sigmoid(cap tanh((zf + bf) / cap)), m_t = max(f + m_(t-1), i) from the slot's kept m (float view [slots, H], left
-    behind); gb [T, 2 H] takes exp(f + m_(t-1) - m_t) and exp(i - m_t), m [T, H] the maxima.  zi, zf float views [T, H]."""
+    behind); gb [T, 2 H] takes exp(f + m_(t-1) - m_t) and exp(i - m_t), m [T, H] the maxima.  zi, zf float views [T, H].  `single_tokens`: every
+    sequence brings one token."""
     _dev("exp_gates", bi, bf, cu_seqlens, slots, gb, m)
     T, H = zi.shape
     for t in (zi, zf):
@@ -1070,9 +1071,9 @@ def exp_gates(zi: torch.Tensor, zf: torch.Tensor, bi: torch.Tensor, bf: torch.Te
     _req(kept.is_cuda and kept.dtype == torch.float32 and kept.dim() == 2 and kept.shape[1] == H and kept.stride(1) == 1, "exp_gates: kept float32 [slots, H]")
     _req(gb.dtype == m.dtype == torch.float32 and gb.shape == (T, 2 * H) and m.shape == (T, H), "exp_gates: gb [T, 2 H], m [T, H] float32")
     _req(cu_seqlens.numel() >= B + 1 and slots.numel() >= B, "exp_gates: arrays shorter than the batch")
-    f = _fn("delta_rule", "br_exp_gates", [_P, _P, c_size_t, _P, _P, c_float, _P, c_size_t, _P, _P, _P, _P, c_int, c_int, _P])
+    f = _fn("delta_rule", "br_exp_gates", [_P, _P, c_size_t, _P, _P, c_float, _P, c_size_t, _P, _P, _P, _P, c_int, c_int, c_int, _P])
     _check(f(_ptr(zi), _ptr(zf), zi.stride(0) if T > 1 else H, _ptr(bi), _ptr(bf), float(cap), _ptr(kept), kept.stride(0), _ptr(cu_seqlens),
-             _ptr(slots), _ptr(gb), _ptr(m), B, H, _stream()), "exp_gates")
+             _ptr(slots), _ptr(gb), _ptr(m), B, H, int(bool(single_tokens)), _stream()), "exp_gates")
 
 
 _DR_FIXED, _DR_DELTA, _DR_WEIGHTED, _DR_CHANNELS = range(4)

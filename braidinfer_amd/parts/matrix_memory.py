@@ -82,7 +82,7 @@ class MatrixMemory(Mixer):
         gb = step.ws.get("mm_gb", (T, 2 * nh), torch.float32)
         m = step.ws.get("mm_m", (T, nh), torch.float32)
         K.exp_gates(rows[:, i0:i0 + nh], rows[:, i0 + nh:], self.b_i, self.b_f, self.cap, ctx.state[:, self.state_floats:], step.cu_seqlens,
-                    step.slots, gb, m, step.n_seqs)
+                    step.slots, gb, m, step.n_seqs, single_tokens=step.is_decode)
         o = step.ws.get("mm_o", (T, he), torch.float32)
         c_out = step.ws.get("mm_c", (T, nh), torch.float32)
         shape = tuple(K.glr_state_shape(nh, d, e + 1))

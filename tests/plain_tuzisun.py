@@ -182,7 +182,7 @@ def window_attention(h, w, p, m, eps, positions):
 def state_space_mixer(h, w, p, m, eps):
     """Mamba-2: gate | inputs | B | C | step sizes in one projection; convolution, state, gate, norm in equal parts."""
     T = h.shape[0]
-    H, e, N, G, parts = m["heads"], m["vdim"], m["state"], m["groups"], m["norm_groups"]
+    H, e, N, G, parts = m["heads"], m["vdim"], m["state"], m.get("groups", 1), m.get("norm_groups", 1)
     inner = H * e
     rows = h @ w[p + "in"].T
     z, xbc, dt = rows[:, :inner], rows[:, inner:2 * inner + 2 * G * N], rows[:, 2 * inner + 2 * G * N:]
@@ -196,8 +196,8 @@ def state_space_mixer(h, w, p, m, eps):
 
 
 def parallel_mixer(h, w, p, m, eps, positions):
-    return (m["left_scale"] * window_attention(h, w, p + "left.", m["left"], eps, positions)
-            + m["right_scale"] * state_space_mixer(h, w, p + "right.", m["right"], eps))
+    return (m.get("left_scale", 1.0) * window_attention(h, w, p + "left.", m["left"], eps, positions)
+            + m.get("right_scale", 1.0) * state_space_mixer(h, w, p + "right.", m["right"], eps))
 
 
 def mlstm_gates(h, w, p, cap):
@@ -209,7 +209,7 @@ def mlstm_gates(h, w, p, cap):
 
 def mlstm_mixer(h, w, p, m, eps, positions):
     T = h.shape[0]
-    H, d, e = m["heads"], m["dim"], m["vdim"]
+    H, d, e = m["heads"], m["dim"], m.get("vdim", m["dim"])
     q = (h @ w[p + "q"].T).reshape(T, H, d) * d ** -0.5
     k, v = (h @ w[p + "k"].T).reshape(T, H, d), (h @ w[p + "v"].T).reshape(T, H, e)
     i, f = mlstm_gates(h, w, p, m["gate_cap"])
@@ -219,7 +219,7 @@ def mlstm_mixer(h, w, p, m, eps, positions):
 
 def channel_delta_mixer(h, w, p, m, eps, positions):
     T = h.shape[0]
-    H, G, d, e = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    H, G, d, e = m["heads"], m.get("kv_heads", m["heads"]), m["dim"], m.get("vdim", m["dim"])
     q = short_convolution(h @ w[p + "q"].T, w[p + "q.conv"]).reshape(T, G, d)
     k = short_convolution(h @ w[p + "k"].T, w[p + "k.conv"]).reshape(T, G, d)
     v = short_convolution(h @ w[p + "v"].T, w[p + "v.conv"]).reshape(T, H, e)
@@ -259,21 +259,24 @@ def connected_half(streams, half, w, c, norm):
     return np.tensordot(w[c + "mix"].T, streams, axes=(1, 0)) + w[c + "out"][:, None, None] * y[None]
 
 
-def forward(cfg, w, tokens, return_layers=False):
-    """Logits [T, vocab] of one sequence from position 0 (and the sum of the streams after every layer)."""
+def forward(cfg, w, tokens, return_layers=False, round_inputs=False):
+    """Logits [T, vocab] of one sequence from position 0 (and the sum of the streams after every layer).  `round_inputs`
+    rounds what every half and the head read to bfloat16 values: how far that alone moves the logits says what a model is
+    worth in bfloat16."""
+    point = (lambda x: to_bf16_values(x)) if round_inputs else (lambda x: x)
     eps = cfg["norm"]["eps"]
-    x = np.repeat(w["embed"][np.asarray(tokens)][None], cfg["streams"], axis=0)
+    x = np.repeat(w["embed"][np.asarray(tokens)][None], cfg.get("streams", 1), axis=0)
     positions = np.arange(len(tokens))
     rows = []
     for i, layer in enumerate(cfg["layers"]):
         p = "l%d." % i
         x = connected_half(x, lambda h: MIXERS[layer["type"]](h, w, p + "mix.", layer["mixer"], eps, positions), w, p + "hc1.",
-                           lambda u: dynamic_tanh(u, w, p + "norm1"))
+                           lambda u: point(dynamic_tanh(u, w, p + "norm1")))
         if layer.get("mlp"):
             x = connected_half(x, lambda h: feed_forward(h, w, p + "mlp.", layer["mlp"]), w, p + "hc2.",
-                               lambda u: dynamic_tanh(u, w, p + "norm2"))
+                               lambda u: point(dynamic_tanh(u, w, p + "norm2")))
         rows.append(x.sum(axis=0))
-    logits = dynamic_tanh(x.sum(axis=0), w, "final.norm") @ w["embed"].T
+    logits = point(dynamic_tanh(x.sum(axis=0), w, "final.norm")) @ w["embed"].T
     return (logits, np.stack(rows)) if return_layers else logits
 
 
@@ -288,7 +291,7 @@ def greedy(cfg, w, prompt, n):
 def tensor_shapes(cfg, ranks=(5, 7)):
     """name -> shape of every tensor of a model of this configuration.  `ranks`: the inner widths of the decay's and the
     gate's low-rank projections, which the tensors alone give."""
-    W, V, s = cfg["width"], cfg["vocab"], cfg["streams"]
+    W, V, s = cfg["width"], cfg["vocab"], cfg.get("streams", 1)
     out = {"embed": (V, W)}
 
     def norm(name):
@@ -309,20 +312,20 @@ def tensor_shapes(cfg, ranks=(5, 7)):
             out[q + "q.norm"] = out[q + "k.norm"] = (d,)
             out[q + "o"], out[q + "o.b"] = (W, H * e), (W,)
             a, q = m["right"], p + "mix.right."
-            inner, bc = a["heads"] * a["vdim"], 2 * a["groups"] * a["state"]
+            inner, bc = a["heads"] * a["vdim"], 2 * a.get("groups", 1) * a["state"]
             out[q + "in"] = (2 * inner + bc + a["heads"], W)
             out[q + "conv"], out[q + "conv.b"] = (inner + bc, a["conv"]), (inner + bc,)
             out[q + "dt_bias"] = out[q + "A_log"] = out[q + "D"] = (a["heads"],)
             out[q + "norm"], out[q + "o"] = (inner,), (W, inner)
         elif layer["type"] == "mlstm":
-            H, d, e = m["heads"], m["dim"], m["vdim"]
+            H, d, e = m["heads"], m["dim"], m.get("vdim", m["dim"])
             out[q + "q"] = out[q + "k"] = (H * d, W)
             out[q + "v"] = out[q + "g"] = (H * e, W)
             out[q + "i"] = out[q + "f"] = (H, W)
             out[q + "i.b"] = out[q + "f.b"] = (H,)
             out[q + "norm"], out[q + "o"] = (H * e,), (W, H * e)
         else:
-            H, G, d, e, n = m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"]
+            H, G, d, e, n = m["heads"], m.get("kv_heads", m["heads"]), m["dim"], m.get("vdim", m["dim"]), m["conv"]
             for x, size in (("q", G * d), ("k", G * d), ("v", H * e)):
                 out[q + x], out[q + x + ".conv"] = (size, W), (size, n)
             out[q + "b"], out[q + "A_log"], out[q + "dt_bias"] = (H, W), (H,), (H * d,)
@@ -352,12 +355,13 @@ def to_bf16_values(a):
     return u.astype(np.uint32).view(np.float32).astype(np.float64).reshape(a32.shape)
 
 
-def random_weights(cfg, seed, gain=1.0, ranks=(5, 7), router_gain=None):
-    """Weights that keep every activation of order one, already rounded to bfloat16.  `gain` sizes the matrices;
-    `router_gain` the router's alone."""
+def random_weights(cfg, seed, gain=1.0, ranks=(5, 7), router_spread=None):
+    """Weights that keep every activation of order one, already rounded to bfloat16.  `gain` sizes the matrices.
+    `router_spread`: the first channel of every feed-forward's input is 1 whatever the token, and the routers read it with
+    weights that far apart and the other channels with small ones, so that a bfloat16 run chooses as the float64 run does."""
     rng = np.random.default_rng(seed)
     w = {}
-    s = cfg["streams"]
+    s = cfg.get("streams", 1)
     for name, shape in tensor_shapes(cfg, ranks).items():
         tail = name.split(".")[-1]
         if tail == "alpha":
@@ -386,11 +390,14 @@ def random_weights(cfg, seed, gain=1.0, ranks=(5, 7), router_gain=None):
             a = 0.3 * rng.standard_normal(shape)
         elif name == "embed":
             a = rng.standard_normal(shape)
-        elif tail == "router" and router_gain is not None:
-            a = rng.standard_normal(shape) * (router_gain / math.sqrt(shape[-1]))
+        elif tail == "router" and router_spread is not None:
+            a = rng.standard_normal(shape) * (0.1 / math.sqrt(shape[-1]))
+            a[:, 0] = router_spread * rng.permutation(shape[0])
         else:
             a = rng.standard_normal(shape) * (1.5 * gain / math.sqrt(shape[-1]))
         w[name] = to_bf16_values(a)
+        if router_spread is not None and ".norm2" in name and shape:
+            w[name][0] = 1.0 if tail == "b" else 0.0
     return w
 
 
