@@ -722,8 +722,8 @@ __global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(const HeadNorm
     }
 }
 
-#define HNG_WIDE_FROM 512      // channels of a row from which a workgroup takes it,
-#define HNG_WIDE_FROM_V4 1025  // and where 16 lanes go four channels at a time
+#define HNG_WIDE_FROM 512      // channels of a row from which a workgroup may take it
+#define HNG_NARROW_ROWS 4096   // rows (of up to 1,024 channels, four at a time) from which 16 lanes a row fill the chip
 
 extern "C" int br_head_norm_gate(const float* o, const float* w, const float* gate, size_t gate_stride, const float* n, const float* m,
                                  float q_mul, void* y, int y_is_bf16, int T, int H, int e, float eps, int gate_sigmoid, int gate_first,
@@ -733,7 +733,7 @@ extern "C" int br_head_norm_gate(const float* o, const float* w, const float* ga
     const size_t n_rows = (size_t)T * H;
     const HeadNormGate p = {o, w, gate, n, m, gate_stride, H, e, gate_sigmoid, gate_first, eps, q_mul};
     const bool v4 = e % 4 == 0 && gate_stride % 4 == 0 && (((uintptr_t)o | (uintptr_t)w | (uintptr_t)gate | (uintptr_t)y) % 16) == 0;
-    if (e >= (v4 ? HNG_WIDE_FROM_V4 : HNG_WIDE_FROM)) {
+    if (e >= HNG_WIDE_FROM && !(v4 && e <= 1024 && n_rows >= HNG_NARROW_ROWS)) {
         if (n_rows > 0x7fffffffULL) return BR_BAD_ARG;
         if (y_is_bf16) head_norm_gate_wide_kernel<bf16><<<(unsigned)n_rows, 256, 0, s>>>(p, (bf16*)y);
         else head_norm_gate_wide_kernel<float><<<(unsigned)n_rows, 256, 0, s>>>(p, (float*)y);

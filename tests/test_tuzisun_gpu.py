@@ -429,12 +429,12 @@ def test_exponential_gates_over_a_running_maximum(H, cap, shift):
     assert float(np.abs(left[:2]).max()) == 0.0 and left[2, 0] == left[2, -1] == 0.0
 
 
-@pytest.mark.parametrize("H,e", [(3, 24), (5, 7), (4, 128), (2, 512), (8, 512), (1, 1100), (2, 515), (6, 1)])
+@pytest.mark.parametrize("T,H,e", [(9, 3, 24), (9, 5, 7), (9, 4, 128), (9, 2, 512), (1030, 4, 512), (9, 1, 1100), (9, 2, 515), (9, 6, 1)])
 @pytest.mark.parametrize("sigmoid", [False, True])
-def test_gate_ahead_of_the_norm_and_the_normaliser(H, e, sigmoid):
+def test_gate_ahead_of_the_norm_and_the_normaliser(T, H, e, sigmoid):
     from braidinfer_amd import kernels as K
     rng = np.random.default_rng(e)
-    T, eps = 9, 1e-3
+    eps = 1e-3
     o, w = f32(rng.standard_normal((T, H, e)) * 0.05), f32(1 + 0.2 * rng.standard_normal(H * e))
     wide = f32(rng.standard_normal((T, H * e + 4)) * 2)
     gate = wide[:, 4:].reshape(T, H, e)
